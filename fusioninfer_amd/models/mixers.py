@@ -35,7 +35,9 @@ model designs assemble them freely:
 * ``LatentAttention``    keys and values expanded from one normed low-rank
   latent per token plus one rotated key part shared by all heads; only the
   latent and the rotated part are cached, the expansions are folded into
-  the queries and the attended latents; optional per-head softmax sink.
+  the queries and the attended latents; optional per-head softmax sink,
+  queries through a normed latent of their own, blended rotary frequencies,
+  a sigmoid gate per head, and layers that read another layer's latents.
 * ``RGLRUMixer``         real-gated linear recurrent unit behind a short
   causal convolution with block-diagonal gates, times a GELU branch.
 * ``SquaredReluMLP``     down(relu(up x)^2) whose up projection may ride a
@@ -60,6 +62,16 @@ model designs assemble them freely:
 * ``PostNormLayer``      x <- x + LN(mixer(x)), x <- x + LN(ff(x)): the
   sublayers read the stream itself and the layer norm (weight and bias)
   sits on their output.
+* ``GatedMemoryMixer``   matrix memory with exponential input and forget
+  gates (capped by a tanh) and a running maximum, fp32 state in the state
+  slots, per-head unit-RMS output with gain and sigmoid gate.
+* ``SharedExpertMoE``    routed experts next to a silu-gated shared expert
+  whose result is multiplied by one sigmoid gate per token; some router
+  outputs may be identity experts.
+* ``HyperLayer``         several copies of the stream: a sublayer reads the
+  RMS norm of a weighted sum of them, and its result is added to every copy
+  while the copies are mixed by a small matrix, all in one kernel with the
+  next sublayer's norm.
 
 Activations run in the model dtype (bf16 or fp32); statistics, rotary
 angles, scores, decays, gates of the recurrence and the state are fp32
@@ -233,18 +245,23 @@ class ParallelMixer(nn.Module):
 
 
 class GatedMLP(nn.Module):
-    """down(act(gate(x)) * up(x)); ``act`` names the fused activation."""
+    """down(act(gate(x)) * up(x)); ``act`` ("gelu_tanh" or "silu") names
+    the fused activation."""
 
     def __init__(self, width: int, ff: int, dtype, act: str = "gelu_tanh"):
         super().__init__()
-        if act != "gelu_tanh":
+        acts = {"gelu_tanh": seqmix.gelu_tanh_and_mul,
+                "silu": seqmix.silu_and_mul}
+        if act not in acts:
             raise ValueError(f"unsupported gated-MLP activation {act!r}")
+        self.ff = ff
+        self._act_and_mul = acts[act]
         self.gate_up_proj = MergedColumnParallelLinear(width, [ff, ff],
                                                        dtype=dtype)
         self.down_proj = RowParallelLinear(ff, width, dtype=dtype)
 
     def forward(self, x):
-        return self.down_proj(seqmix.gelu_tanh_and_mul(self.gate_up_proj(x)))
+        return self.down_proj(self._act_and_mul(self.gate_up_proj(x)))
 
 
 class MixerLayer(nn.Module):
@@ -488,8 +505,13 @@ class RoutedExperts(nn.Module):
     keep) the router is group-limited: sigmoid scores, the choice runs on
     score + a per-expert correction inside the ``keep`` best of ``count``
     groups of neighbouring experts, and the weights are the chosen scores
-    as they are. On the GPU the experts run
-    as two grouped GEMMs over block-aligned expert segments: the MFMA
+    as they are. With ``identity`` not None the router has that many further
+    outputs after the experts': scores are softmax over all of them, the
+    choice runs on score + correction, weights are the chosen scores as they
+    are, and a chosen identity expert returns the input itself (it has no
+    weights and runs no product; see ``route_identity``). ``side_gates``
+    further router rows are plain scalar gates of the input that ride the
+    same fp32 product. On the GPU the experts run as two grouped GEMMs over block-aligned expert segments: the MFMA
     kernel on packed bf16 weights where the sizes fit its tiles, the
     plain grouped kernel otherwise (fp32, odd sizes)."""
 
@@ -497,7 +519,8 @@ class RoutedExperts(nn.Module):
                  score: str = "sigmoid", renorm: bool = True,
                  scale: float = 1.0, act: str = "silu_gate",
                  router_bias: bool = False, limit: float = 0.0,
-                 groups: Optional[Tuple[int, int]] = None):
+                 groups: Optional[Tuple[int, int]] = None,
+                 identity: Optional[int] = None, side_gates: int = 0):
         super().__init__()
         if score not in ("sigmoid", "softmax"):
             raise ValueError(f"unknown router score {score!r}")
@@ -515,19 +538,33 @@ class RoutedExperts(nn.Module):
                     f"router groups {groups} do not fit {experts} experts "
                     f"with top {top}")
             self.groups = (count, keep)
-        if not 1 <= top <= experts:
-            raise ValueError("top must be in 1..experts")
+        self.identity = identity
+        self.outputs = experts + (identity or 0)   # what the router chooses from
+        self.side_gates = int(side_gates)
+        if identity is not None:
+            if groups is not None or score != "softmax" or renorm \
+                    or scale != 1.0:
+                raise ValueError("identity experts go with plain softmax "
+                                 "scores")
+            if identity < 0:
+                raise ValueError("identity must not be negative")
+        elif side_gates:
+            raise ValueError("side gates go with identity routing")
+        if not 1 <= top <= self.outputs:
+            raise ValueError("top must be in 1..router outputs")
         self.width, self.ff, self.experts, self.top = width, ff, experts, top
         self.score, self.renorm, self.scale = score, renorm, float(scale)
         self.dtype = dtype
         self.router = nn.Parameter(
-            torch.empty(experts, width, dtype=torch.float32).normal_(0, 0.02),
+            torch.empty(self.outputs + self.side_gates, width,
+                        dtype=torch.float32).normal_(0, 0.02),
             requires_grad=False)
         self.router_bias = (_f32_param((experts,), 0.0) if router_bias
                             else None)
-        # group-limited routing: added to the scores for the choice only
-        self.correction = (_f32_param((experts,), 0.0)
-                           if self.groups is not None else None)
+        # added to the scores for the choice only
+        self.correction = (_f32_param((self.outputs,), 0.0)
+                           if self.groups is not None or identity is not None
+                           else None)
         # gated: gate rows then up rows; otherwise the up rows alone
         self.gate_up = nn.Parameter(
             torch.empty(experts, (2 if self.gated else 1) * ff, width,
@@ -577,11 +614,30 @@ class RoutedExperts(nn.Module):
         return ops.moe_route(logits, self.top, self.score, self.renorm,
                              self.scale)
 
+    def route_identity(self, x):
+        """(weights, ids, weight of the identity experts [T], scalar gates'
+        logits [T, side_gates] fp32) with ``identity`` routing."""
+        from fusioninfer_amd import ops
+
+        logits = F.linear(x.float(), self.router)
+        topv, topi, idw = ops.moe_route_corrected(
+            logits[:, : self.outputs], self.correction, self.top,
+            self.experts)
+        return topv, topi, idw, logits[:, self.outputs:]
+
     def forward(self, x: torch.Tensor) -> torch.Tensor:
+        if self.identity is not None:
+            topv, topi, idw, _ = self.route_identity(x)
+            y = self.run_experts(x, topv, topi).float()
+            return (y + idw[:, None] * x.float()).to(x.dtype)
+        return self.run_experts(x, *self.route(x))
+
+    def run_experts(self, x, topv, topi) -> torch.Tensor:
+        """Weighted sum of the chosen experts (ids beyond ``experts`` add
+        nothing)."""
         from fusioninfer_amd import ops
 
         T = x.shape[0]
-        topv, topi = self.route(x)
         if not x.is_cuda:
             out = torch.zeros(T, self.width, dtype=torch.float32)
             for e in range(self.experts):
@@ -725,6 +781,13 @@ class LatentAttentionConfig:
     sink: bool = True        # learned per-head term in the denominator
     rot_dims: int = -1       # leading entries of the rotated part that turn
                              # (-1: all of it)
+    q_rank: int = 0          # >0: queries come from a normed latent
+    head_gate: bool = False  # sigmoid gate per head on the result
+    # frequency blend for context extension (rot_original 0: none)
+    rot_factor: float = 1.0
+    rot_original: float = 0.0
+    rot_fast: float = 0.0
+    rot_slow: float = 0.0
 
     def __post_init__(self):
         if self.rot_dims < 0:
@@ -800,69 +863,125 @@ class TemperedGatedAttention(nn.Module):
 
 
 class LatentAttention(nn.Module):
-    """q and the down projection (latent | shared rotated key part) come
-    from the merged projection. The key expansion is folded into the
-    queries (q_h^T W_uk,h) and the value expansion applied to the attended
-    latents, so attention runs over the cached rows [latent | rotated
-    part] with one shared key/value head."""
+    """The query projection (or its latent), the down projection (latent |
+    shared rotated key part) and the head gate come from the merged
+    projection. The key expansion is folded into the queries
+    (q_h^T W_uk,h) and the value expansion applied to the attended latents,
+    so attention runs over the cached rows [latent | rotated part] with one
+    shared key/value head. With ``own_kv`` False the block has no down
+    projection and ``forward`` is handed the cache of the layer it borrows
+    from."""
 
     has_bias = False
 
     def __init__(self, cfg: LatentAttentionConfig, width: int, eps: float,
-                 dtype):
+                 dtype, own_kv: bool = True):
         super().__init__()
         self.cfg = cfg
         self.eps = eps
         self.dtype = dtype
+        self.own_kv = own_kv
         H = cfg.heads
-        self.in_sizes = [H * (cfg.dim + cfg.rot_dim), cfg.rank + cfg.rot_dim]
-        self.in_names = ["q", "dkv"]
-        self.c_norm = _f32_param((cfg.rank,), 1.0)
+        q_size = H * (cfg.dim + cfg.rot_dim)
+        if cfg.q_rank:
+            self.in_names, self.in_sizes = ["dq"], [cfg.q_rank]
+            self.q_norm = _f32_param((cfg.q_rank,), 1.0)
+            self.uq = ReplicatedLinear(cfg.q_rank, q_size, dtype=dtype)
+        else:
+            self.in_names, self.in_sizes = ["q"], [q_size]
+            self.q_norm = self.uq = None
+        self.c_norm = None
+        if own_kv:
+            self.in_names.append("dkv")
+            self.in_sizes.append(cfg.rank + cfg.rot_dim)
+            self.c_norm = _f32_param((cfg.rank,), 1.0)
+        if cfg.head_gate:
+            self.in_names.append("g")
+            self.in_sizes.append(H)
         self.uk = nn.Parameter(
             torch.empty(H * cfg.dim, cfg.rank, dtype=dtype).normal_(0, 0.02),
             requires_grad=False)
-        self.uv = nn.Parameter(
-            torch.empty(H * cfg.vdim, cfg.rank, dtype=dtype).normal_(0, 0.02),
+        # kept [H, rank, vdim]: the right operand of the batched product
+        # must be dense as it stands
+        self.uv_t = nn.Parameter(
+            torch.empty(H, cfg.rank, cfg.vdim, dtype=dtype).normal_(0, 0.02),
             requires_grad=False)
         self.sink = _f32_param((H,), 0.0) if cfg.sink else None
         self.o_proj = RowParallelLinear(H * cfg.vdim, width, dtype=dtype)
-        self.register_buffer(
-            "inv_freq", rotary_inv_freq(cfg.rot_dims, cfg.rot_base),
-            persistent=False)
+        inv_freq, mult = seqmix.blended_rotary(
+            cfg.rot_dims, cfg.rot_base, cfg.rot_factor, cfg.rot_original,
+            cfg.rot_fast, cfg.rot_slow)
+        self.rot_mult = float(mult)
+        self.register_buffer("inv_freq", inv_freq, persistent=False)
+
+    @property
+    def uv(self) -> torch.Tensor:
+        """The value expansion as [H * vdim, rank]."""
+        c = self.cfg
+        return self.uv_t.transpose(1, 2).reshape(c.heads * c.vdim, c.rank)
 
     def state_tensors(self, num_blocks, block_size, num_slots, device):
+        if not self.own_kv:
+            return {}
         c = self.cfg
         return {"kv": torch.zeros(
             (num_blocks, 1, block_size, c.rank + c.rot_dim),
             dtype=self.dtype, device=device)}
 
     def block_bytes(self, block_size: int) -> int:
+        if not self.own_kv:
+            return 0
         c = self.cfg
         esize = torch.empty((), dtype=self.dtype).element_size()
         return block_size * (c.rank + c.rot_dim) * esize
 
-    def forward(self, parts, meta, cache) -> torch.Tensor:
-        q, dkv = parts
+    def _queries(self, parts, meta, cache):
+        """Latent rows into the cache; returns (unfolded queries
+        [T, H*(dim+rot_dim)], folded query buffer with its rotated part
+        filled)."""
         c = self.cfg
-        T, H = q.shape[0], c.heads
-        qf = torch.empty((T, H, c.rank + c.rot_dim), dtype=q.dtype,
-                         device=q.device)
-        seqmix.latent_rope_cache_(
-            q, dkv, meta.positions, self.inv_freq, self.c_norm, self.eps,
-            cache["kv"], meta.slot_mapping, H, c.dim, c.rot_dim, c.rank, qf)
+        H = c.heads
+        q, dkv = parts.get("q"), parts.get("dkv")
+        T = next(iter(parts.values())).shape[0]
+        dev = self.uk.device
+        qf = torch.empty((T, H, c.rank + c.rot_dim), dtype=self.dtype,
+                         device=dev)
+        if not c.q_rank and self.own_kv and self.rot_mult == 1.0:
+            seqmix.latent_rope_cache_(
+                q, dkv, meta.positions, self.inv_freq, self.c_norm, self.eps,
+                cache["kv"], meta.slot_mapping, H, c.dim, c.rot_dim, c.rank,
+                qf)
+            return q, qf
+        if c.q_rank or self.own_kv:
+            cq = seqmix.latent_norm_cache_(
+                parts.get("dq"), dkv, meta.positions, self.inv_freq,
+                self.rot_mult, self.q_norm, self.c_norm, self.eps,
+                cache["kv"], meta.slot_mapping, c.rank, c.rot_dim)
+            if c.q_rank:
+                q = self.uq(cq)
+        seqmix.latent_query_rope_(q, meta.positions, self.inv_freq,
+                                  self.rot_mult, H, c.dim, c.rot_dim, c.rank,
+                                  qf)
+        return q, qf
+
+    def forward(self, parts, meta, cache) -> torch.Tensor:
+        parts = dict(zip(self.in_names, parts))
+        c = self.cfg
+        H = c.heads
+        q, qf = self._queries(parts, meta, cache)
+        T = q.shape[0]
         # fold the key expansion into the queries: [H, T, dim] x [H, dim, rank]
         qu = q.view(T, H, c.dim + c.rot_dim)[:, :, : c.dim].transpose(0, 1)
         torch.bmm(qu, self.uk.view(H, c.dim, c.rank),
                   out=qf.transpose(0, 1)[:, :, : c.rank])
         o = seqmix.sink_paged_attention(
             qf, cache["kv"], None, meta.seq_bt, meta.row_seq, meta.positions,
-            c.scale, sink=self.sink, value_dims=c.rank, seq_cu=meta.seq_cu,
+            c.scale, sink=self.sink, value_dims=c.rank,
+            out_gate=parts.get("g"), seq_cu=meta.seq_cu,
             tiles=meta.seq_tiles)
         # expand the attended latents: [H, T, rank] x [H, rank, vdim]
         ov = torch.empty((T, H, c.vdim), dtype=q.dtype, device=q.device)
-        torch.bmm(o.transpose(0, 1),
-                  self.uv.view(H, c.vdim, c.rank).transpose(1, 2),
-                  out=ov.transpose(0, 1))
+        torch.bmm(o.transpose(0, 1), self.uv_t, out=ov.transpose(0, 1))
         return self.o_proj(ov.view(T, H * c.vdim))
 
 
@@ -1151,3 +1270,147 @@ class PostNormLayer(nn.Module):
             return x
         return seqmix.post_norm_residual_(resid, self.mlp(x), self.norm2,
                                           self.norm2_b, self.eps, self.dtype)
+
+
+# ------------------------------------------------------------------------
+# Family of blocks around several copies of the stream
+
+
+@dataclasses.dataclass
+class GatedMemoryConfig:
+    heads: int
+    dim: int                 # per-head query/key size
+    vdim: int                # per-head value size
+    gate_cap: float          # tanh cap of both gate inputs
+
+    def __post_init__(self):
+        if self.gate_cap <= 0:
+            raise ValueError("gate_cap must be positive")
+
+
+class GatedMemoryMixer(nn.Module):
+    """Matrix memory: q, k, v, output gate and the two gates' inputs come
+    from the merged projection (the gate biases are added in fp32)."""
+
+    has_bias = False
+
+    def __init__(self, cfg: GatedMemoryConfig, width: int, eps: float, dtype):
+        super().__init__()
+        self.cfg = cfg
+        self.eps = eps
+        self.dtype = dtype
+        H, n, nv = cfg.heads, cfg.heads * cfg.dim, cfg.heads * cfg.vdim
+        self.in_sizes = [n, n, nv, nv, H, H]
+        self.in_names = ["q", "k", "v", "g", "i", "f"]
+        self.i_bias = _f32_param((H,), 0.0)
+        self.f_bias = _f32_param((H,), 0.0)
+        self.norm_w = _f32_param((nv,), 1.0)
+        self.o_proj = RowParallelLinear(nv, width, dtype=dtype)
+
+    def state_tensors(self, num_blocks, block_size, num_slots, device):
+        c = self.cfg
+        return {
+            "mem": torch.zeros((num_slots, c.heads, c.dim, c.vdim),
+                               dtype=torch.float32, device=device),
+            "aux": torch.zeros(
+                (num_slots, c.heads, seqmix.memory_state_copies(c.vdim),
+                 c.dim + 1), dtype=torch.float32, device=device),
+        }
+
+    def block_bytes(self, block_size: int) -> int:
+        return 0
+
+    def forward(self, parts, meta, cache) -> torch.Tensor:
+        q, k, v, g, i, f = parts
+        c = self.cfg
+        o_raw = seqmix.gated_memory(
+            q, k, v, i, f, self.i_bias, self.f_bias, c.gate_cap,
+            cache["mem"], cache["aux"], meta.seq_cu, meta.seq_slots,
+            meta.positions, c.heads, c.dim, c.vdim, tiles=meta.seq_tiles)
+        o = seqmix.group_rms_gate(o_raw, g, self.norm_w, c.heads, self.eps,
+                                  "sigmoid", self.dtype)
+        return self.o_proj(o)
+
+
+class SharedExpertMoE(nn.Module):
+    """sum of the chosen experts + identity weight * h + sigmoid(w h) *
+    shared(h). ``terms`` hands the summands to the caller's residual kernel
+    with their per-row coefficients."""
+
+    def __init__(self, routed: RoutedExperts, shared: Optional[GatedMLP]):
+        super().__init__()
+        if routed.identity is None:
+            raise ValueError("needs identity routing (identity may be 0)")
+        if (shared is not None) != (routed.side_gates == 1):
+            raise ValueError("a shared expert takes one scalar gate")
+        self.routed = routed
+        self.shared = shared
+
+    def terms(self, h):
+        r = self.routed
+        topv, topi, idw, side = r.route_identity(h)
+        out = [(r.run_experts(h, topv, topi), None, False)]
+        if self.shared is not None:
+            out.append((self.shared(h), side[:, 0], True))
+        if r.identity:
+            out.append((h, idw, False))
+        return out
+
+
+class HyperLayer(nn.Module):
+    """``streams`` fp32 copies x_s of the residual stream. Per sublayer,
+    with vectors a (in), b (out) and a matrix M of its own:
+
+        y = sublayer(rms(sum_s a_s x_s) * w);  x_t <- sum_s M[s,t] x_s + b_t y
+
+    Every update is fused with the read and the norm of the sublayer that
+    follows: ``forward`` receives this layer's normed input and the (in
+    vector, norm weight) of what comes next, and returns the next normed
+    input. The mixer's input branches are one merged projection."""
+
+    def __init__(self, mixer: nn.Module, mlp: Optional[nn.Module],
+                 streams: int, width: int, eps: float, dtype):
+        super().__init__()
+        self.mixer = mixer
+        self.mlp = mlp
+        self.eps = eps
+        self.dtype = dtype
+        self.branches: List[str] = list(mixer.in_names)
+        self.sizes: List[int] = list(mixer.in_sizes)
+        self.in_proj = MergedColumnParallelLinear(
+            width, self.sizes, dtype=dtype, bias=mixer.has_bias)
+
+        def copies():
+            return (_f32_param((streams,), 1.0 / streams),
+                    _f32_param((streams,), 1.0),
+                    nn.Parameter(torch.eye(streams, dtype=torch.float32),
+                                 requires_grad=False))
+
+        self.norm1 = _f32_param((width,), 1.0)
+        self.hc1_in, self.hc1_out, self.hc1_mix = copies()
+        if mlp is not None:
+            self.norm2 = _f32_param((width,), 1.0)
+            self.hc2_in, self.hc2_out, self.hc2_mix = copies()
+
+    def in_proj_rows(self, branch: str):
+        off = 0
+        for name, size in zip(self.branches, self.sizes):
+            if name == branch:
+                return off, size
+            off += size
+        raise KeyError(branch)
+
+    def forward(self, xs, h, meta, cache, nxt):
+        parts = self.in_proj(h).split(self.sizes, dim=-1)
+        y = self.mixer(parts, meta, cache)
+        w_in, norm_w = ((self.hc2_in, self.norm2) if self.mlp is not None
+                        else nxt)
+        h = seqmix.hyper_update_(xs, [(y, None, False)], self.hc1_mix,
+                                 self.hc1_out, w_in, norm_w, self.eps,
+                                 self.dtype)
+        if self.mlp is None:
+            return h
+        terms = (self.mlp.terms(h) if hasattr(self.mlp, "terms")
+                 else [(self.mlp(h), None, False)])
+        return seqmix.hyper_update_(xs, terms, self.hc2_mix, self.hc2_out,
+                                    nxt[0], nxt[1], self.eps, self.dtype)

@@ -356,7 +356,7 @@ class MomedraLM(nn.Module):
             elif isinstance(mod, LatentAttention):
                 out[mp + "dkv.norm"] = (mod.c_norm, None)
                 out[mp + "uk"] = (mod.uk, None)
-                out[mp + "uv"] = (mod.uv, None)
+                out[mp + "uv"] = (mod.uv_t, ("heads_t",))
                 if mod.sink is not None:
                     out[mp + "sink"] = (mod.sink, None)
             else:
@@ -391,6 +391,8 @@ class MomedraLM(nn.Module):
         dst = param.data
         if spec is None:
             return dst
+        if spec[0] == "heads_t":     # stored [H, in, out] per head
+            return dst.transpose(1, 2)
         if spec[0] == "cols":        # [B, a:a+n, ...] of a stacked tensor
             return dst[:, spec[1]: spec[1] + spec[2]]
         if spec[0] == "idx":
@@ -407,6 +409,9 @@ class MomedraLM(nn.Module):
             raise ValueError(f"unknown tensor {name!r}")
         param, spec = names[name]
         dst = self._view(param, spec)
+        if spec is not None and spec[0] == "heads_t" and \
+                t.shape == (dst.shape[0] * dst.shape[1], dst.shape[2]):
+            t = t.view(dst.shape)
         if dst.shape != t.shape:
             raise ValueError(f"{name}: shape {tuple(t.shape)} does not fit "
                              f"{tuple(dst.shape)}")
@@ -415,8 +420,13 @@ class MomedraLM(nn.Module):
     def export_weights(self) -> Dict[str, torch.Tensor]:
         """Inverse of load_weights (checkpoint naming), for writing
         random-init models to disk."""
-        return {k: self._view(p, spec).detach().clone().contiguous()
-                for k, (p, spec) in self._name_map().items()}
+        out = {}
+        for k, (p, spec) in self._name_map().items():
+            t = self._view(p, spec).detach().clone().contiguous()
+            if spec is not None and spec[0] == "heads_t":
+                t = t.view(-1, t.shape[-1])
+            out[k] = t
+        return out
 
     def randomize_small_params(self, seed: int = 0) -> None:
         """Random-init use (benchmarks, tests): give gains, biases, sinks,

@@ -280,6 +280,19 @@ def _register_builtin_architectures() -> None:
     register_architecture("Kazozen", kazozen_config, kazozen_model,
                           extensions=("seqmix", "moe"))
 
+    def sufavik_config(raw, model_path):
+        from fusioninfer_amd.models import sufavik
+
+        return sufavik.model_config_from_dict(raw, model_path)
+
+    def sufavik_model(cfg):
+        from fusioninfer_amd.models.sufavik import SufavikLM
+
+        return SufavikLM(cfg)
+
+    register_architecture("Sufavik", sufavik_config, sufavik_model,
+                          extensions=("seqmix", "moe"))
+
 
 _register_builtin_architectures()
 

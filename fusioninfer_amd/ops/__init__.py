@@ -529,6 +529,29 @@ def moe_route_grouped(logits: torch.Tensor, correction: torch.Tensor,
     return ref.moe_route_grouped(logits, correction, k, groups, keep)
 
 
+def moe_route_corrected(logits: torch.Tensor, correction: torch.Tensor,
+                        k: int, experts: int):
+    """Router tail with a choice correction and identity experts: s =
+    softmax(logits) in fp32 over all columns (``logits`` may be the leading
+    columns of a wider row), the k largest s + correction chosen (ties:
+    smaller index), weights = the chosen s, not renormalised. Ids from
+    ``experts`` on are identity experts; their weights are summed per row.
+    Returns (weights [T,k] fp32, ids [T,k] int32, identity weight [T])."""
+    E = logits.shape[1]
+    if not 1 <= k <= E or not 1 <= experts <= E:
+        raise ValueError("top and experts must be within the router's rows")
+    if logits.is_cuda:
+        T = logits.shape[0]
+        dev = logits.device
+        topv = torch.empty(T, k, dtype=torch.float32, device=dev)
+        topi = torch.empty(T, k, dtype=torch.int32, device=dev)
+        idw = torch.empty(T, dtype=torch.float32, device=dev)
+        _moe_native().moe_route_corrected(logits, correction, topv, topi,
+                                          idw, k, experts)
+        return topv, topi, idw
+    return ref.moe_route_corrected(logits, correction, k, experts)
+
+
 def moe_combine(out, y, pos, w):
     """out[t] = sum_k w[t,k] * y[pos[t,k]] (pos < 0 skipped). Deterministic
     (no atomics) so token-exact tests stay reproducible. bf16 or fp32

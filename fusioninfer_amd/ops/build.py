@@ -3,7 +3,7 @@
 Drives hipcc directly — no CUDA compatibility layer, no JIT cache: the
 resulting ``_C.so`` lives next to this file so the gpurun snapshot carries it.
 
-Two extensions, so that a model family compiles only what it runs:
+Three extensions, so that a model family compiles only what it runs:
 
   core    -> _C.so         transformer kernels
   seqmix  -> _C_seqmix.so  sequence-mixer kernels (ops/seqmix.py)
@@ -18,6 +18,7 @@ import os
 import subprocess
 import sys
 import sysconfig
+from concurrent.futures import ThreadPoolExecutor
 
 OPS_DIR = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(OPS_DIR, "csrc")
@@ -52,11 +53,14 @@ SEQMIX_SOURCES = [
     "seqmix_parallel.hip",
     "seqmix_sink.hip",
     "seqmix_postnorm.hip",
+    "seqmix_hyper.hip",
+    "seqmix_memory.hip",
+    "seqmix_hyper_bindings.hip",
 ]
 
 EXTENSIONS = {
     "core": ("_C", SOURCES, ["common.h"]),
-    "seqmix": ("_C_seqmix", SEQMIX_SOURCES, ["common.h", "seqmix.h"]),
+    "seqmix": ("_C_seqmix", SEQMIX_SOURCES, ["common.h", "seqmix.h", "seqmix_bind.h", "seqmix_hyper.h"]),
     "moe": ("_C_moe", MOE_SOURCES, ["common.h", "seqmix.h"]),
 }
 
@@ -76,25 +80,20 @@ def build_extension(ext: str, verbose: bool = True,
     from torch.utils import cpp_extension as ce
 
     mod_name, sources, headers = EXTENSIONS[ext]
-    SO_PATH = extension_path(ext)
+    so_path = extension_path(ext)
     srcs = [os.path.join(CSRC, s) for s in sources]
     hdrs = [os.path.join(CSRC, h) for h in headers]
-    if not force and os.path.exists(SO_PATH):
-        so_mtime = os.path.getmtime(SO_PATH)
+    if not force and os.path.exists(so_path):
+        so_mtime = os.path.getmtime(so_path)
         if all(os.path.getmtime(f) < so_mtime for f in srcs + hdrs):
-            return SO_PATH
-    # build next to the target and rename: a concurrent reader never sees
-    # a half-written library
-    final_path, SO_PATH = SO_PATH, SO_PATH + ".%d.tmp" % os.getpid()
-
+            return so_path
     hipcc = os.path.join(os.environ.get("ROCM_PATH", "/opt/rocm"), "bin", "hipcc")
     torch_lib = ce.library_paths()[0]
-    cmd = [
+    common = [
         hipcc,
         "--offload-arch=gfx950",
         "-O3",
         "-std=c++17",
-        "-shared",
         "-fPIC",
         f"-DTORCH_EXTENSION_NAME={mod_name}",
         # packed-fp32 VALU forms are kept out of generated code
@@ -106,7 +105,42 @@ def build_extension(ext: str, verbose: bool = True,
         *[f"-I{p}" for p in ce.include_paths()],
         f"-I{sysconfig.get_paths()['include']}",
         f"-I{CSRC}",
-        *srcs,
+    ]
+    out = None if verbose else subprocess.DEVNULL
+
+    def run(cmd):
+        if verbose:
+            print("[fusioninfer build]", " ".join(cmd), file=sys.stderr)
+        subprocess.run(cmd, check=True, stdout=out, stderr=out)
+
+    # one object per source, compiled side by side; objects newer than their
+    # source and all headers are kept unless ``force``
+    obj_dir = os.path.join(OPS_DIR, "build", ext)
+    os.makedirs(obj_dir, exist_ok=True)
+    newest_hdr = max(os.path.getmtime(f) for f in hdrs)
+
+    def compile_one(src):
+        obj = os.path.join(obj_dir, os.path.basename(src) + ".o")
+        if not force and os.path.exists(obj) and os.path.getmtime(obj) > max(
+                os.path.getmtime(src), newest_hdr):
+            return obj
+        tmp = obj + ".%d.tmp" % os.getpid()
+        run(common + ["-c", src, "-o", tmp])
+        os.replace(tmp, obj)
+        return obj
+
+    jobs = int(os.environ.get("MAX_JOBS") or min(os.cpu_count() or 1, 8))
+    with ThreadPoolExecutor(max_workers=max(1, min(jobs, 16))) as pool:
+        objs = list(pool.map(compile_one, srcs))
+    # link next to the target and rename: a concurrent reader never sees a
+    # half-written library
+    tmp = so_path + ".%d.tmp" % os.getpid()
+    run([
+        hipcc,
+        "--offload-arch=gfx950",
+        "-shared",
+        "-fPIC",
+        *objs,
         f"-L{torch_lib}",
         f"-Wl,-rpath,{torch_lib}",
         "-ltorch",
@@ -116,15 +150,10 @@ def build_extension(ext: str, verbose: bool = True,
         "-lc10_hip",
         "-lamdhip64",
         "-o",
-        SO_PATH,
-    ]
-    if verbose:
-        print("[fusioninfer build]", " ".join(cmd), file=sys.stderr)
-    subprocess.run(cmd, check=True,
-                   stdout=None if verbose else subprocess.DEVNULL,
-                   stderr=None if verbose else subprocess.DEVNULL)
-    os.replace(SO_PATH, final_path)
-    return final_path
+        tmp,
+    ])
+    os.replace(tmp, so_path)
+    return so_path
 
 
 if __name__ == "__main__":

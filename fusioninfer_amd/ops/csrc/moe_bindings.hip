@@ -16,6 +16,9 @@ void launch_moe_gemm(u16*, const u16*, const u16*, const int*, const int*,
                      const int*, int, int, int, int, int, float, hipStream_t);
 void launch_moe_route_grouped(const float*, const float*, float*, int*, int,
                               int, int, int, int, hipStream_t);
+void launch_moe_route_corrected(const float*, int64_t, const float*, float*,
+                                int*, float*, int, int, int, int,
+                                hipStream_t);
 void launch_moe_gemm_fp8(u16*, const unsigned char*, const float*,
                          const unsigned char*, const float*, const int*,
                          const int*, const int*, int, int, int, int, bool,
@@ -217,6 +220,33 @@ void moe_route_grouped(at::Tensor logits, at::Tensor correction,
       (int)keep, current_stream());
 }
 
+void moe_route_corrected(at::Tensor logits, at::Tensor correction,
+                         at::Tensor topv, at::Tensor topi,
+                         at::Tensor id_weight, int64_t k, int64_t experts) {
+  TORCH_CHECK(logits.is_cuda() && logits.scalar_type() == at::kFloat &&
+              logits.dim() == 2 &&
+              (logits.stride(1) == 1 || logits.size(1) == 1));
+  TORCH_CHECK(correction.is_cuda() && correction.scalar_type() == at::kFloat &&
+              correction.is_contiguous());
+  TORCH_CHECK(topv.scalar_type() == at::kFloat && topv.is_contiguous() &&
+              topi.scalar_type() == at::kInt && topi.is_contiguous() &&
+              id_weight.scalar_type() == at::kFloat &&
+              id_weight.is_contiguous());
+  const int T = logits.size(0);
+  const int E = logits.size(1);
+  TORCH_CHECK(correction.numel() == E);
+  TORCH_CHECK(E >= 1 && E <= 1024 && k >= 1 && k <= E && experts >= 1 &&
+              experts <= E, "moe_route_corrected: 1 <= k <= outputs <= 1024");
+  TORCH_CHECK(topv.numel() == T * k && topi.numel() == T * k &&
+              id_weight.numel() == T);
+  if (T == 0) return;
+  fi::launch_moe_route_corrected(
+      logits.data_ptr<float>(), logits.stride(0),
+      correction.data_ptr<float>(), topv.data_ptr<float>(),
+      topi.data_ptr<int>(), id_weight.data_ptr<float>(), T, E, (int)k,
+      (int)experts, current_stream());
+}
+
 void moe_route(at::Tensor logits, at::Tensor topv, at::Tensor topi, int64_t k,
                bool sigmoid, bool renorm, double scale) {
   TORCH_CHECK(logits.is_cuda() && logits.scalar_type() == at::kFloat &&
@@ -290,6 +320,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("moe_route_grouped", &moe_route_grouped,
         "group-limited router tail: sigmoid scores, choice on score + "
         "correction inside the best groups, weights = chosen scores");
+  m.def("moe_route_corrected", &moe_route_corrected,
+        "softmax router tail: choice on score + correction, weights = chosen "
+        "scores, identity experts' weights summed per token");
   m.def("moe_route", &moe_route,
         "router tail for any expert count: softmax/sigmoid scores, top-k, "
         "renormalize, constant factor");

@@ -22,6 +22,10 @@
 //    is the sum of its two largest choice scores, the best `keep` groups
 //    stay, and the k largest c inside them are chosen (ties: smaller
 //    index). Weights are the chosen s as they are.
+//  * moe_route_corrected: softmax scores s over all columns; the k largest
+//    s + correction are chosen (ties: smaller index), weights are the
+//    chosen s as they are. Columns from `experts` on are identity experts,
+//    whose chosen weights are also summed per token.
 //  * moe_combine: out[t] = sum_k w[t,k] * y[pos[t,k]], any width, bf16 or
 //    fp32 rows, no atomics.
 
@@ -194,6 +198,77 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(
   }
 }
 
+__global__ __launch_bounds__(256) void moe_route_corrected_kernel(
+    const float* __restrict__ logits, const int64_t l_stride,
+    const float* __restrict__ correction, float* __restrict__ topv,
+    int* __restrict__ topi, float* __restrict__ id_weight, const int T,
+    const int E, const int k, const int experts) {
+  const int t = blockIdx.x * 4 + threadIdx.x / kWaveSize;
+  if (t >= T) return;
+  const int lane = threadIdx.x % kWaveSize;
+  const float* row = logits + t * l_stride;
+  float s[kRouteSlots];
+  float m = -INFINITY;
+#pragma unroll
+  for (int j = 0; j < kRouteSlots; ++j) {
+    const int e = lane + 64 * j;
+    s[j] = e < E ? row[e] : -INFINITY;
+    m = fmaxf(m, s[j]);
+  }
+  m = wave_reduce_max(m);
+  float sum = 0.f;
+#pragma unroll
+  for (int j = 0; j < kRouteSlots; ++j) {
+    s[j] = lane + 64 * j < E ? expf(s[j] - m) : 0.f;
+    sum += s[j];
+  }
+  sum = wave_reduce_sum(sum);
+  float c[kRouteSlots];
+#pragma unroll
+  for (int j = 0; j < kRouteSlots; ++j) {
+    const int e = lane + 64 * j;
+    s[j] /= sum;
+    c[j] = e < E ? s[j] + correction[e] : 0.f;
+  }
+  unsigned taken = 0;      // bit j: slot j of this lane is already chosen
+  float idw = 0.f;
+  for (int it = 0; it < k; ++it) {
+    float v = -INFINITY, sv = 0.f;
+    int idx = 0x7fffffff;
+#pragma unroll
+    for (int j = 0; j < kRouteSlots; ++j) {
+      const int e = lane + 64 * j;
+      // ascending j: the smaller index wins ties
+      if (e < E && !((taken >> j) & 1u) && (idx == 0x7fffffff || c[j] > v)) {
+        v = c[j];
+        sv = s[j];
+        idx = e;
+      }
+    }
+#pragma unroll
+    for (int off = 32; off; off >>= 1) {
+      const float ov = __shfl_xor(v, off);
+      const float os = __shfl_xor(sv, off);
+      const int oi = __shfl_xor(idx, off);
+      if (oi != 0x7fffffff &&
+          (idx == 0x7fffffff || ov > v || (ov == v && oi < idx))) {
+        v = ov;
+        sv = os;
+        idx = oi;
+      }
+    }
+    if (lane == 0) {
+      topi[static_cast<int64_t>(t) * k + it] = idx;
+      topv[static_cast<int64_t>(t) * k + it] = sv;
+    }
+    if (idx >= experts) idw += sv;
+#pragma unroll
+    for (int j = 0; j < kRouteSlots; ++j)
+      if (idx == lane + 64 * j) taken |= 1u << j;
+  }
+  if (lane == 0) id_weight[t] = idw;
+}
+
 constexpr int kPlainBM = 16;   // rows per workgroup
 constexpr int kPlainBN = 64;   // columns per workgroup
 constexpr int kPlainKT = 32;   // K step
@@ -313,6 +388,15 @@ void launch_moe_route_grouped(const float* logits, const float* correction,
   hipLaunchKernelGGL(moe_route_grouped_kernel, dim3(ceil_div(T, 4)),
                      dim3(256), 0, stream, logits, correction, topv, topi, T,
                      E, k, groups, keep);
+}
+
+void launch_moe_route_corrected(const float* logits, int64_t l_stride,
+                                const float* correction, float* topv,
+                                int* topi, float* id_weight, int T, int E,
+                                int k, int experts, hipStream_t stream) {
+  hipLaunchKernelGGL(moe_route_corrected_kernel, dim3(ceil_div(T, 4)),
+                     dim3(256), 0, stream, logits, l_stride, correction, topv,
+                     topi, id_weight, T, E, k, experts);
 }
 
 template <typename A>

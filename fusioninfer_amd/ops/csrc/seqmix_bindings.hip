@@ -3,12 +3,8 @@
 // assume before launching.
 
 #include <algorithm>
-#include <torch/extension.h>
 
-#include <c10/hip/HIPStream.h>
-#include <hip/hip_runtime.h>
-
-#include "seqmix.h"
+#include "seqmix_bind.h"
 
 namespace fi {
 template <typename A>
@@ -162,46 +158,7 @@ void launch_tanh_cap(float*, int64_t, float, hipStream_t);
 
 namespace {
 
-using fi::u16;
-
-hipStream_t stream() { return c10::hip::getCurrentHIPStream().stream(); }
-
-bool is_act(const at::Tensor& t) {
-  return t.scalar_type() == at::kFloat || t.scalar_type() == at::kBFloat16;
-}
-
-#define CHECK_ACT(t)                                                 \
-  TORCH_CHECK((t).is_cuda(), #t " must be on the GPU");              \
-  TORCH_CHECK(is_act(t), #t " must be float32 or bfloat16")
-#define CHECK_F32(t)                                                  \
-  TORCH_CHECK((t).is_cuda() && (t).scalar_type() == at::kFloat &&     \
-                  (t).is_contiguous(),                                \
-              #t " must be a contiguous float32 GPU tensor")
-#define CHECK_I32(t)                                                  \
-  TORCH_CHECK((t).is_cuda() && (t).scalar_type() == at::kInt &&       \
-                  (t).is_contiguous(),                                \
-              #t " must be a contiguous int32 GPU tensor")
-
-// rows of a 2-D activation view whose last dim is dense
-void check_rows(const at::Tensor& t, int64_t T, int64_t n, const char* what) {
-  TORCH_CHECK(t.dim() == 2 && t.size(0) == T && t.size(1) == n &&
-                  (t.stride(1) == 1 || n == 1),
-              what, ": expected [", T, ", ", n, "] with dense rows");
-}
-
-#define DISPATCH_ACT(t, ...)                          \
-  if ((t).scalar_type() == at::kFloat) {              \
-    using A = float;                                  \
-    __VA_ARGS__;                                      \
-  } else {                                            \
-    using A = u16;                                    \
-    __VA_ARGS__;                                      \
-  }
-
-template <typename A>
-A* ptr(const at::Tensor& t) {
-  return reinterpret_cast<A*>(t.data_ptr());
-}
+using namespace fi_bind;
 
 void scalar_rms_norm(at::Tensor out, at::Tensor x, at::Tensor g, double eps) {
   CHECK_ACT(out);
@@ -1325,6 +1282,7 @@ void tanh_cap(at::Tensor x, double cap) {
 
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  register_hyper_ops(m);
   m.def("pair_embed", &pair_embed,
         "embedding times a constant plus a (previous id, id) table row; the "
         "previous id of a group's first row lives in a slot state");

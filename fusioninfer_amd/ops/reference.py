@@ -404,6 +404,18 @@ def moe_route_grouped(logits, correction, k: int, groups: int, keep: int):
     return s.gather(1, topi), topi.int()
 
 
+def moe_route_corrected(logits, correction, k: int, experts: int):
+    """Scores s = softmax over all columns; the k largest s + correction
+    are chosen with weights s as they are. Columns from ``experts`` on are
+    identity experts: their chosen weights are also summed per row.
+    Returns (weights, ids, identity weight [T])."""
+    s = torch.softmax(logits.float(), dim=-1)
+    topi = (s + correction.float()).topk(k, dim=-1).indices
+    topv = s.gather(1, topi)
+    idw = (topv * (topi >= experts)).sum(-1)
+    return topv, topi.int(), idw
+
+
 def moe_route(logits, k: int, score: str, renorm: bool, scale: float):
     """Router tail: softmax or sigmoid scores, top-k, optional division by
     the chosen scores' sum (+1e-20), constant factor."""

@@ -600,3 +600,111 @@ def tanh_cap_(logits, cap: float):
         _native().tanh_cap(logits, float(cap))
         return logits
     return ref.tanh_cap_(logits, cap)
+
+
+# ------------------------------------------------------------------------
+# several copies of the stream mixed by small matrices, latent attention
+# with a query latent, matrix memory with exponential gates, silu product
+
+def hyper_start(ids, embed, w_in, norm_w, eps: float, act_dtype):
+    """All copies of the stream start as embed[id]; returns (copies
+    [T, S, W] fp32, rms(sum_s w_in[s] copy_s) * norm_w)."""
+    if embed.is_cuda:
+        T, W, S = ids.shape[0], embed.shape[1], w_in.numel()
+        xs = torch.empty((T, S, W), dtype=torch.float32, device=embed.device)
+        h = torch.empty((T, W), dtype=act_dtype, device=embed.device)
+        _native().hyper_start(xs, h, ids, embed, w_in, norm_w, eps)
+        return xs, h
+    return ref.hyper_start(ids, embed, w_in, norm_w, eps, act_dtype)
+
+
+def hyper_update_(xs, terms, mix, w_out, w_in, norm_w, eps: float, out_dtype):
+    """Copies of the stream (fp32 [T, S, W], in place): copy t <- sum_s
+    mix[s, t] copy_s + w_out[t] * y, all from the old ones; returns the
+    next sublayer's input rms(sum_s w_in[s] copy_s) * norm_w. y is the sum
+    of one to three terms (rows [T, W], coefficient, sigmoid): coefficient
+    None or one fp32 number per row (any stride), passed through a sigmoid
+    first if asked."""
+    if not 1 <= len(terms) <= 3:
+        raise ValueError("one to three terms")
+    if xs.is_cuda:
+        h = torch.empty((xs.shape[0], xs.shape[2]), dtype=out_dtype,
+                        device=xs.device)
+        ts = list(terms) + [(None, None, False)] * (3 - len(terms))
+        flat = [x for rows, coef, sig in ts for x in (rows, coef, bool(sig))]
+        _native().hyper_update(xs, h, *flat, mix, w_out, w_in, norm_w, eps)
+        return h
+    return ref.hyper_update_(xs, terms, mix, w_out, w_in, norm_w, eps,
+                             out_dtype)
+
+
+def latent_norm_cache_(dq, dkv, positions, inv_freq, rot_mult: float, q_w,
+                       c_w, eps: float, kv_cache, slot_mapping, rank: int,
+                       rot_dim: int):
+    """dq (or None): returned RMS-normed with q_w, contiguous. dkv (or
+    None): [normed latent | rotated part] into the paged cache. Both may be
+    column slices of one projection output."""
+    src = dq if dq is not None else dkv
+    if src is not None and src.is_cuda:
+        out = None
+        if dq is not None:
+            out = torch.empty(dq.shape, dtype=dq.dtype, device=dq.device)
+        _native().latent_norm_cache(out, dq, dkv, positions, inv_freq,
+                                    float(rot_mult), q_w, c_w, eps, kv_cache,
+                                    slot_mapping, int(rank), int(rot_dim))
+        return out
+    return ref.latent_norm_cache_(dq, dkv, positions, inv_freq, rot_mult,
+                                  q_w, c_w, eps, kv_cache, slot_mapping,
+                                  rank, rot_dim)
+
+
+def latent_query_rope_(q, positions, inv_freq, rot_mult: float,
+                       num_heads: int, dim: int, rot_dim: int, rank: int,
+                       q_out):
+    """Rotated trailing part of every query head into q_out[:, :, rank:]
+    ([T, H, rank+rot_dim])."""
+    if q.is_cuda:
+        _native().latent_query_rope(q_out, q, positions, inv_freq,
+                                    float(rot_mult), num_heads, dim, rot_dim,
+                                    rank)
+        return
+    ref.latent_query_rope_(q, positions, inv_freq, rot_mult, num_heads, dim,
+                           rot_dim, rank, q_out)
+
+
+MEMORY_COLUMNS = 64  # value columns per workgroup of the memory kernels
+
+
+def memory_state_copies(vdim: int) -> int:
+    """Copies of (normalizer, maximum) per head: every workgroup of a head
+    reads and writes its own."""
+    return (vdim + MEMORY_COLUMNS - 1) // MEMORY_COLUMNS
+
+
+def gated_memory(q, k, v, ilin, flin, i_bias, f_bias, cap: float, mem, aux,
+                 seq_cu, seq_slots, positions, heads: int, dim: int,
+                 vdim: int, tiles=None):
+    """Read-outs (fp32 [T, heads*vdim]) of the matrix memory with
+    exponential gates. q/k/v/ilin/flin may be column slices of one
+    projection output. ``tiles`` as for ranged_paged_attention: the leading
+    row groups that are prompt portions."""
+    if q.is_cuda:
+        T = q.shape[0]
+        out = torch.empty((T, heads * vdim), dtype=torch.float32,
+                          device=q.device)
+        _native().gated_memory(out, q, k, v, ilin, flin, i_bias, f_bias,
+                               float(cap), mem, aux, seq_cu, seq_slots,
+                               positions, heads, dim, vdim)
+        return out
+    return ref.gated_memory(q, k, v, ilin, flin, i_bias, f_bias, cap, mem,
+                            aux, seq_cu, seq_slots, positions, heads, dim,
+                            vdim)
+
+
+def silu_and_mul(gu):
+    if gu.is_cuda:
+        out = torch.empty((gu.shape[0], gu.shape[1] // 2), dtype=gu.dtype,
+                          device=gu.device)
+        _native().silu_and_mul(out, gu)
+        return out
+    return ref.silu_and_mul(gu)

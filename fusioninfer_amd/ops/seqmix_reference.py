@@ -475,11 +475,11 @@ def headnorm_qtemp_cache_(q, k, v, positions, q_w, k_w, eps: float,
     return qf.to(q.dtype)
 
 
-def _rotate_interleaved(x, ang):
-    """Pairs (2i, 2i+1) of the last dim of x turned by ang[..., i]; pairs
-    beyond the angles given pass unchanged."""
+def _rotate_interleaved(x, ang, mult: float = 1.0):
+    """Pairs (2i, 2i+1) of the last dim of x turned by ang[..., i], cos and
+    sin times ``mult``; pairs beyond the angles given pass unchanged."""
     n = 2 * ang.shape[-1]
-    cs, sn = torch.cos(ang), torch.sin(ang)
+    cs, sn = torch.cos(ang) * mult, torch.sin(ang) * mult
     u, w = x[..., 0:n:2], x[..., 1:n:2]
     out = x.clone()
     out[..., 0:n:2] = u * cs - w * sn
@@ -769,3 +769,129 @@ def tanh_cap_(logits, cap: float):
     """logits (fp32, in place) <- cap * tanh(logits / cap)."""
     logits.copy_(cap * torch.tanh(logits / cap))
     return logits
+
+
+# ------------------------------------------------------------------------
+# several copies of the stream mixed by small matrices, latent attention
+# with a query latent, matrix memory with exponential gates, silu product
+
+def hyper_start(ids, embed, w_in, norm_w, eps: float, act_dtype):
+    """Every copy of the stream starts as embed[id]. Returns (copies
+    [T, S, W] fp32, rms(sum_s w_in[s] copy_s) * norm_w in act_dtype)."""
+    x = embed[ids.long()].float()
+    S = w_in.numel()
+    xs = x[:, None, :].expand(-1, S, -1).contiguous()
+    u = (xs * w_in.float()[None, :, None]).sum(1)
+    return xs, (_rms(u, eps) * norm_w.float()).to(act_dtype)
+
+
+def hyper_update_(xs, terms, mix, w_out, w_in, norm_w, eps: float, out_dtype):
+    """xs [T, S, W] fp32, in place: copy t <- sum_s mix[s, t] copy_s +
+    w_out[t] * y with y = sum of the terms (rows, coefficient, sigmoid?):
+    coefficient None or fp32 [T], passed through a sigmoid if asked. Then
+    returns rms(sum_s w_in[s] copy_s) * norm_w."""
+    y = None
+    for rows, coef, sig in terms:
+        v = rows.float()
+        if coef is not None:
+            c = coef.float()
+            v = v * (torch.sigmoid(c) if sig else c)[:, None]
+        y = v if y is None else y + v
+    new = torch.einsum("st,nsw->ntw", mix.float(), xs)
+    new = new + w_out.float()[None, :, None] * y[:, None, :]
+    xs.copy_(new)
+    u = (new * w_in.float()[None, :, None]).sum(1)
+    return (_rms(u, eps) * norm_w.float()).to(out_dtype)
+
+
+def latent_norm_cache_(dq, dkv, positions, inv_freq, rot_mult: float, q_w,
+                       c_w, eps: float, kv_cache, slot_mapping, rank: int,
+                       rot_dim: int):
+    """dq [T, q_rank] (or None): returned RMS-normed with q_w. dkv
+    [T, rank+rot_dim] (or None): leading part RMS-normed with c_w, trailing
+    part rotated (cos/sin times rot_mult), the row goes to the paged
+    kv_cache [B, 1, bs, rank+rot_dim]."""
+    if dkv is not None:
+        ang = positions.float()[:, None] * inv_freq.float()[None, :]
+        cf = dkv.float()
+        row = torch.cat([_rms(cf[:, :rank], eps) * c_w.float(),
+                         _rotate_interleaved(cf[:, rank:], ang, rot_mult)],
+                        dim=-1)
+        bs = kv_cache.shape[2]
+        slots = slot_mapping.long()
+        ok = slots >= 0
+        kv_cache[slots[ok] // bs, 0, slots[ok] % bs, :] = row[ok].to(
+            kv_cache.dtype)
+    if dq is None:
+        return None
+    return (_rms(dq.float(), eps) * q_w.float()).to(dq.dtype)
+
+
+def latent_query_rope_(q, positions, inv_freq, rot_mult: float,
+                       num_heads: int, dim: int, rot_dim: int, rank: int,
+                       q_out):
+    """q [T, H*(dim+rot_dim)]: the trailing rot_dim entries of every head
+    turned (cos/sin times rot_mult) into q_out[:, :, rank:]."""
+    T = q.shape[0]
+    ang = positions.float()[:, None] * inv_freq.float()[None, :]
+    qr = q.float().reshape(T, num_heads, dim + rot_dim)[:, :, dim:]
+    q_out[:, :, rank:] = _rotate_interleaved(
+        qr, ang[:, None, :], rot_mult).to(q_out.dtype)
+
+
+def memory_gates(ilin, flin, i_bias, f_bias, cap: float):
+    """(log input gate, log forget gate) [T, H] fp32:
+    cap * tanh((i + b) / cap) and log sigmoid(cap * tanh((f + b) / cap))."""
+    li = cap * torch.tanh((ilin.float() + i_bias.float()) / cap)
+    lf = torch.nn.functional.logsigmoid(
+        cap * torch.tanh((flin.float() + f_bias.float()) / cap))
+    return li, lf
+
+
+def gated_memory(q, k, v, ilin, flin, i_bias, f_bias, cap: float, mem, aux,
+                 seq_cu, seq_slots, positions, heads: int, dim: int,
+                 vdim: int):
+    """Matrix memory with exponential gates. Per head, with log gates i, f
+    and a running maximum m (0 before the first token):
+
+        m_t = max(f + m_(t-1), i)
+        S <- exp(f + m_(t-1) - m_t) S + exp(i - m_t) k v^T,  n alike with k
+        o = S^T q' / (max(|n . q'|, exp(-m_t)) + 1e-6),  q' = dim^-1/2 q.
+
+    ``mem`` [slots, H, dim, vdim] fp32 keeps S, ``aux`` [slots, H, copies,
+    dim+1] fp32 keeps n and m (equal copies). Returns fp32 [T, H*vdim]."""
+    T = q.shape[0]
+    qf = q.float().reshape(T, heads, dim) * dim ** -0.5
+    kf = k.float().reshape(T, heads, dim)
+    vf = v.float().reshape(T, heads, vdim)
+    li, lf = memory_gates(ilin, flin, i_bias, f_bias, cap)
+    o = torch.empty(T, heads, vdim, dtype=torch.float32)
+    cu, slots, pos = seq_cu.tolist(), seq_slots.tolist(), positions.tolist()
+    for s in range(len(slots)):
+        a, b = cu[s], cu[s + 1]
+        if b <= a:
+            continue
+        S = _group_state(mem, slots[s], pos[a], (heads, dim, vdim))
+        nm = (_group_state(aux[:, :, 0], slots[s], pos[a], (heads, dim + 1)))
+        n, m = nm[:, :dim].clone(), nm[:, dim].clone()
+        for t in range(a, b):
+            m_new = torch.maximum(lf[t] + m, li[t])
+            keep = torch.exp(lf[t] + m - m_new)
+            add = torch.exp(li[t] - m_new)
+            S = (keep[:, None, None] * S + add[:, None, None]
+                 * kf[t][:, :, None] * vf[t][:, None, :])
+            n = keep[:, None] * n + add[:, None] * kf[t]
+            m = m_new
+            den = torch.maximum((n * qf[t]).sum(-1).abs(), torch.exp(-m))
+            o[t] = (torch.einsum("hij,hi->hj", S, qf[t])
+                    / (den + 1e-6)[:, None])
+        if slots[s] >= 0:
+            mem[slots[s]] = S
+            aux[slots[s]] = torch.cat([n, m[:, None]], dim=1)[:, None, :]
+    return o.reshape(T, heads * vdim)
+
+
+def silu_and_mul(gu):
+    """gu: [T, 2F] (gate | up) -> silu(gate) * up."""
+    g, u = gu.float().chunk(2, dim=-1)
+    return (torch.nn.functional.silu(g) * u).to(gu.dtype)
