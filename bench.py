@@ -72,16 +72,15 @@ def parse_args():
                         "workload mode; headline stays spec-off)")
     p.add_argument("--mixer-compare", action="store_true",
                    help="instead of the serving benchmark: prefill and "
-                        "decode token throughput of the Kazozen, Momedra, "
-                        "Sefalorn and Pinuvik designs at real-model layer "
-                        "sizes (random "
-                        "weights) next to the Qwen3-style transformer of "
+                        "decode token throughput of the Sufavik, Kazozen, "
+                        "Momedra, Sefalorn and Pinuvik designs at "
+                        "real-model layer sizes (random weights) next to the Qwen3-style transformer of "
                         "the same sizes")
     p.add_argument("--mc-sizes", default="2048x16,4096x32",
                    help="WIDTHxHEADS list for --mixer-compare (head dim "
                         "128, kv heads = heads/4, ff = 3*width)")
     p.add_argument("--mc-archs",
-                   default="kazozen,momedra,sefalorn,pinuvik,transformer")
+                   default="sufavik,kazozen,momedra,sefalorn,pinuvik,transformer")
     p.add_argument("--mc-layers", type=int, default=4)
     p.add_argument("--mc-prompt", type=int, default=2048)
     p.add_argument("--mc-prefill-seqs", type=int, default=4)
@@ -105,6 +104,36 @@ def _mixer_compare_config(arch, width, heads, layers, chunk, vocab=32000):
         mc.hidden_size, mc.num_layers = width, layers
         mc.num_heads, mc.num_kv_heads, mc.head_dim = heads, kv, dim
         mc.intermediate_size, mc.vocab_size = ff, vocab
+        return mc
+    if arch == "sufavik":
+        # two copies of the stream; latent attention with a dense and with
+        # a routed feed-forward, the matrix memory, and a latent layer that
+        # reads the second layer's latents, in turn; the routed layers'
+        # active size (shared + top * ff) equals the dense ff
+        moe = {"kind": "moe", "expert": {"ff": ff // 4},
+               "router": {"experts": 8, "identity": 2, "top": 2},
+               "shared": {"ff": ff // 2}}
+        dense = {"kind": "dense", "ff": ff}
+        latent = {"heads": heads, "dim": 96, "rot_dim": 32, "vdim": dim,
+                  "kv_rank": 256, "q_rank": 3 * width // 8,
+                  "scale": dim ** -0.5,
+                  "rot": {"base": 1e6, "dims": 32,
+                          "scaling": {"factor": 4.0, "original": 4096,
+                                      "fast": 32.0, "slow": 1.0}}}
+        memory = {"heads": heads, "dim": dim, "vdim": dim, "gate_cap": 15.0}
+        raw_layers = []
+        for i in range(layers):
+            u = i % 4
+            mixer = dict(memory if u == 2 else latent)
+            if u == 3:
+                mixer["kv_from"] = i - 2
+            raw_layers.append({
+                "type": "mlstm" if u == 2 else "latent_attention",
+                "mixer": mixer, "mlp": dense if u == 0 else moe})
+        raw = {"architecture": "Sufavik", "vocab": vocab, "width": width,
+               "norm": {"eps": 1e-5}, "streams": 2, "layers": raw_layers}
+        mc = model_config_from_dict(raw)
+        mc.name = f"sufavik-{width}x{heads}"
         return mc
     if arch == "kazozen":
         # windowed sink attention with 4 kept first keys; every second

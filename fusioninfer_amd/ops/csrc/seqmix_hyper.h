@@ -61,4 +61,18 @@ void launch_gated_memory_scan(float* out, MemoryInputs<A> in, float* mem,
                               int s0, int S, int H, int D, int V,
                               hipStream_t st);
 
+// groups 0 .. groups-1 (the ones the tile table covers) in chunks; scratch:
+// chunk_mem [2 tiles, H, ceil(V/64), 64, 16 row_tiles], chunk_n [2 tiles, H,
+// 16 row_tiles], meta [2 tiles, H, 3]
+bool gated_memory_has_chunks(int D);
+int gated_memory_row_tiles(int D);
+template <typename A>
+void launch_gated_memory_chunks(float* out, float* chunk_mem, float* chunk_n,
+                                double* meta, MemoryInputs<A> in, float* mem,
+                                float* aux, const int* seq_cu,
+                                const int* seq_slots, const int* positions,
+                                const int* tile_seq, const int* tile_row0,
+                                int tiles, int groups, int H, int D, int V,
+                                hipStream_t st);
+
 }  // namespace fi

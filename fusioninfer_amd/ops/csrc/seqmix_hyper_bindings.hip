@@ -181,7 +181,8 @@ void gated_memory(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v,
                   at::Tensor i, at::Tensor f, at::Tensor i_bias,
                   at::Tensor f_bias, double cap, at::Tensor mem,
                   at::Tensor aux, at::Tensor seq_cu, at::Tensor seq_slots,
-                  at::Tensor positions, int64_t H, int64_t D, int64_t V) {
+                  at::Tensor positions, int64_t H, int64_t D, int64_t V,
+                  OptTensor tile_seq, OptTensor tile_row0, int64_t tile_rows) {
   CHECK_ACT(q);
   CHECK_F32(out);
   CHECK_F32(i_bias);
@@ -213,13 +214,40 @@ void gated_memory(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v,
   const int S = seq_slots.numel();
   TORCH_CHECK(seq_cu.numel() == S + 1 && positions.numel() == T);
   if (T == 0) return;
+  // leading groups in chunks: all rows past tile_rows are one-row groups
+  int groups = 0, tiles = 0;
+  at::Tensor chunk_mem, chunk_n, meta;
+  if (tile_seq.has_value() && fi::gated_memory_has_chunks((int)D)) {
+    CHECK_I32(*tile_seq);
+    TORCH_CHECK(tile_row0.has_value());
+    CHECK_I32(*tile_row0);
+    TORCH_CHECK(tile_row0->numel() == tile_seq->numel());
+    TORCH_CHECK(tile_rows >= 0 && tile_rows <= T && S >= T - tile_rows);
+    groups = S - (int)(T - tile_rows);
+    tiles = tile_seq->numel();
+    TORCH_CHECK(2 * tiles <= 65535 && groups <= 65535);
+    const int64_t dp = 16 * fi::gated_memory_row_tiles((int)D);
+    const auto f32 = q.options().dtype(at::kFloat);
+    chunk_mem = at::empty({2 * tiles * H * copies * fi::kMemoryCols * dp}, f32);
+    chunk_n = at::empty({2 * tiles * H * dp}, f32);
+    meta = at::empty({2 * tiles * H * 3}, q.options().dtype(at::kDouble));
+  }
   DISPATCH_ACT(q, {
     const auto in = memory_inputs<A>(q, k, v, i, f, i_bias, f_bias, cap);
+    if (groups > 0)
+      fi::launch_gated_memory_chunks<A>(
+          out.data_ptr<float>(), chunk_mem.data_ptr<float>(),
+          chunk_n.data_ptr<float>(), meta.data_ptr<double>(), in,
+          mem.data_ptr<float>(), aux.data_ptr<float>(),
+          seq_cu.data_ptr<int>(), seq_slots.data_ptr<int>(),
+          positions.data_ptr<int>(), tile_seq->data_ptr<int>(),
+          tile_row0->data_ptr<int>(), tiles, groups, (int)H, (int)D, (int)V,
+          stream());
     fi::launch_gated_memory_scan<A>(
         out.data_ptr<float>(), in, mem.data_ptr<float>(),
         aux.data_ptr<float>(), seq_cu.data_ptr<int>(),
-        seq_slots.data_ptr<int>(), positions.data_ptr<int>(), 0, S, (int)H,
-        (int)D, (int)V, stream());
+        seq_slots.data_ptr<int>(), positions.data_ptr<int>(), groups, S,
+        (int)H, (int)D, (int)V, stream());
   });
 }
 

@@ -692,9 +692,14 @@ def gated_memory(q, k, v, ilin, flin, i_bias, f_bias, cap: float, mem, aux,
         T = q.shape[0]
         out = torch.empty((T, heads * vdim), dtype=torch.float32,
                           device=q.device)
+        tile_seq = tile_row0 = None
+        tile_rows = 0
+        if tiles is not None and tiles[2] > 0:
+            tile_seq, tile_row0, tile_rows = tiles
         _native().gated_memory(out, q, k, v, ilin, flin, i_bias, f_bias,
                                float(cap), mem, aux, seq_cu, seq_slots,
-                               positions, heads, dim, vdim)
+                               positions, heads, dim, vdim, tile_seq,
+                               tile_row0, int(tile_rows))
         return out
     return ref.gated_memory(q, k, v, ilin, flin, i_bias, f_bias, cap, mem,
                             aux, seq_cu, seq_slots, positions, heads, dim,
