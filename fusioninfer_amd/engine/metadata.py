@@ -38,6 +38,10 @@ class AttnMetadata:
     # tile table over the prefill groups for tiled sequence-mixer kernels
     # (ops.seqmix.build_attention_tiles); None on all-decode steps
     seq_tiles: Optional[tuple] = None
+    # host view of the prefill groups: (new rows, context length after the
+    # step, block ids) per group; and what ops.seqmix.context_rows made of it
+    prefill_spans: Optional[list] = None
+    context_rows: object = None
     # LoRA groups for this step (fusioninfer_amd.lora.LoRABatch) or None
     lora: object = None
 

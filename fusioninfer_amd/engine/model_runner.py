@@ -249,6 +249,9 @@ class ModelRunner:
 
             meta.seq_tiles = seqmix.build_attention_tiles(
                 prefill_payload["new_lens"], device=dev)
+            meta.prefill_spans = list(zip(
+                prefill_payload["new_lens"], prefill_payload["total_lens"],
+                prefill_payload["bt"]))
         return meta
 
     def _lora_batch(self, prefill_payload, decode_payload, np_=0):

@@ -868,7 +868,9 @@ class LatentAttention(nn.Module):
     projection. The key expansion is folded into the queries
     (q_h^T W_uk,h) and the value expansion applied to the attended latents,
     so attention runs over the cached rows [latent | rotated part] with one
-    shared key/value head. With ``own_kv`` False the block has no down
+    shared key/value head. Prompt portions long enough to pay for it gather
+    their contexts' rows and attend over expanded per-head keys and values
+    instead (less than half the products). With ``own_kv`` False the block has no down
     projection and ``forward`` is handed the cache of the layer it borrows
     from."""
 
@@ -906,6 +908,7 @@ class LatentAttention(nn.Module):
         self.uv_t = nn.Parameter(
             torch.empty(H, cfg.rank, cfg.vdim, dtype=dtype).normal_(0, 0.02),
             requires_grad=False)
+        self._expand_w = None
         self.sink = _f32_param((H,), 0.0) if cfg.sink else None
         self.o_proj = RowParallelLinear(H * cfg.vdim, width, dtype=dtype)
         inv_freq, mult = seqmix.blended_rotary(
@@ -935,53 +938,123 @@ class LatentAttention(nn.Module):
         esize = torch.empty((), dtype=self.dtype).element_size()
         return block_size * (c.rank + c.rot_dim) * esize
 
-    def _queries(self, parts, meta, cache):
-        """Latent rows into the cache; returns (unfolded queries
-        [T, H*(dim+rot_dim)], folded query buffer with its rotated part
-        filled)."""
-        c = self.cfg
-        H = c.heads
-        q, dkv = parts.get("q"), parts.get("dkv")
-        T = next(iter(parts.values())).shape[0]
-        dev = self.uk.device
-        qf = torch.empty((T, H, c.rank + c.rot_dim), dtype=self.dtype,
-                         device=dev)
-        if not c.q_rank and self.own_kv and self.rot_mult == 1.0:
-            seqmix.latent_rope_cache_(
-                q, dkv, meta.positions, self.inv_freq, self.c_norm, self.eps,
-                cache["kv"], meta.slot_mapping, H, c.dim, c.rot_dim, c.rank,
-                qf)
-            return q, qf
-        if c.q_rank or self.own_kv:
-            cq = seqmix.latent_norm_cache_(
-                parts.get("dq"), dkv, meta.positions, self.inv_freq,
-                self.rot_mult, self.q_norm, self.c_norm, self.eps,
-                cache["kv"], meta.slot_mapping, c.rank, c.rot_dim)
-            if c.q_rank:
-                q = self.uq(cq)
-        seqmix.latent_query_rope_(q, meta.positions, self.inv_freq,
-                                  self.rot_mult, H, c.dim, c.rot_dim, c.rank,
-                                  qf)
-        return q, qf
+    # prompt portions attend over expanded keys and values once an average
+    # context row is read by this many new rows ...
+    expand_rows_per_key = 64
+    # ... as long as the expansions stay within this many bytes
+    expand_max_bytes = 4 << 30
 
-    def forward(self, parts, meta, cache) -> torch.Tensor:
-        parts = dict(zip(self.in_names, parts))
+    def _expands(self, meta) -> bool:
+        """Whether the step's prompt portions attend in expanded form."""
         c = self.cfg
-        H = c.heads
-        q, qf = self._queries(parts, meta, cache)
-        T = q.shape[0]
+        spans = meta.prefill_spans
+        if not spans or meta.seq_tiles is None:
+            return False
+        if not seqmix.expansion_pays(spans, self.expand_rows_per_key):
+            return False
+        esize = torch.empty((), dtype=self.dtype).element_size()
+        per_row = c.heads * (c.dim + c.rot_dim + c.vdim) * esize
+        if per_row * sum(n for _, n, _ in spans) > self.expand_max_bytes:
+            return False
+        return (self.uk.device.type != "cuda" or seqmix.attention_has_tiles(
+            c.dim + c.rot_dim, c.vdim))
+
+    def invalidate_packed(self):
+        """The expansion weights changed (checkpoint load, tests)."""
+        self._expand_w = None
+
+    def _expand_weights(self):
+        """Matrices that turn a cached row [latent | rotated part] into all
+        heads' keys [unrotated | rotated], and its latent into all heads'
+        values. The rotated part is copied by unit rows."""
+        if self._expand_w is None:
+            c = self.cfg
+            H, N = c.heads, c.rank + c.rot_dim
+            wk = torch.zeros((H, c.dim + c.rot_dim, N), dtype=self.dtype,
+                             device=self.uk.device)
+            wk[:, : c.dim, : c.rank] = self.uk.data.view(H, c.dim, c.rank)
+            wk[:, c.dim:, c.rank:] = torch.eye(
+                c.rot_dim, dtype=self.dtype, device=self.uk.device)
+            self._expand_w = (wk.view(-1, N), self.uv.contiguous())
+        return self._expand_w
+
+    def _attend_expanded(self, q, gate, meta, cache, out):
+        """q: unfolded contiguous queries of the prompt portions' rows,
+        rotated in place; result rows [*, H, vdim] into ``out``."""
+        c = self.cfg
+        R, H, D = q.shape[0], c.heads, c.dim + c.rot_dim
+        kv = cache["kv"]
+        if meta.context_rows is None:
+            meta.context_rows = seqmix.ContextRows(
+                meta.prefill_spans, kv.shape[2], kv.device)
+        ctx = meta.context_rows
+        pos = meta.positions[:R]
+        qh = q.view(R, H, D)
+        seqmix.latent_query_rope_(q, pos, self.inv_freq, self.rot_mult, H,
+                                  c.dim, c.rot_dim, c.dim, qh)
+        wk, wv = self._expand_weights()
+        rows = seqmix.paged_rows_gather(kv, ctx.slots)
+        k = F.linear(rows, wk).view(ctx.count, H, 1, D)
+        v = F.linear(rows[:, : c.rank], wv).view(ctx.count, H, 1, c.vdim)
+        n = len(meta.prefill_spans)
+        seqmix.sink_paged_attention(
+            qh, k, v, ctx.table, meta.row_seq[:R], pos, c.scale,
+            sink=self.sink, out_gate=gate, seq_cu=meta.seq_cu[: n + 1],
+            tiles=meta.seq_tiles, out=out)
+
+    def _attend_folded(self, q, qf, gate, meta, cache, row0, out):
+        """Rows row0.. with the expansions folded around the attention; qf
+        holds their rotated query parts."""
+        c = self.cfg
+        T, H = q.shape[0], c.heads
         # fold the key expansion into the queries: [H, T, dim] x [H, dim, rank]
         qu = q.view(T, H, c.dim + c.rot_dim)[:, :, : c.dim].transpose(0, 1)
         torch.bmm(qu, self.uk.view(H, c.dim, c.rank),
                   out=qf.transpose(0, 1)[:, :, : c.rank])
         o = seqmix.sink_paged_attention(
-            qf, cache["kv"], None, meta.seq_bt, meta.row_seq, meta.positions,
-            c.scale, sink=self.sink, value_dims=c.rank,
-            out_gate=parts.get("g"), seq_cu=meta.seq_cu,
-            tiles=meta.seq_tiles)
+            qf, cache["kv"], None, meta.seq_bt, meta.row_seq[row0:],
+            meta.positions[row0:], c.scale, sink=self.sink,
+            value_dims=c.rank, out_gate=gate, seq_cu=meta.seq_cu,
+            tiles=meta.seq_tiles if row0 == 0 else None)
         # expand the attended latents: [H, T, rank] x [H, rank, vdim]
+        torch.bmm(o.transpose(0, 1), self.uv_t, out=out.transpose(0, 1))
+
+    def forward(self, parts, meta, cache) -> torch.Tensor:
+        parts = dict(zip(self.in_names, parts))
+        c = self.cfg
+        H, g = c.heads, parts.get("g")
+        T = meta.positions.shape[0]
+        R = meta.seq_tiles[2] if self._expands(meta) else 0
+        q, dkv, qf = parts.get("q"), parts.get("dkv"), None
+        if R < T:
+            qf = torch.empty((T - R, H, c.rank + c.rot_dim),
+                             dtype=self.dtype, device=self.uk.device)
+        if (R == 0 and not c.q_rank and self.own_kv
+                and self.rot_mult == 1.0):
+            seqmix.latent_rope_cache_(
+                q, dkv, meta.positions, self.inv_freq, self.c_norm, self.eps,
+                cache["kv"], meta.slot_mapping, H, c.dim, c.rot_dim, c.rank,
+                qf)
+        else:
+            if c.q_rank or self.own_kv:
+                cq = seqmix.latent_norm_cache_(
+                    parts.get("dq"), dkv, meta.positions, self.inv_freq,
+                    self.rot_mult, self.q_norm, self.c_norm, self.eps,
+                    cache["kv"], meta.slot_mapping, c.rank, c.rot_dim)
+                if c.q_rank:
+                    q = self.uq(cq)
+            if R < T:
+                seqmix.latent_query_rope_(
+                    q[R:], meta.positions[R:], self.inv_freq, self.rot_mult,
+                    H, c.dim, c.rot_dim, c.rank, qf)
         ov = torch.empty((T, H, c.vdim), dtype=q.dtype, device=q.device)
-        torch.bmm(o.transpose(0, 1), self.uv_t, out=ov.transpose(0, 1))
+        if R > 0:
+            self._attend_expanded(q[:R].contiguous(),
+                                  g[:R] if g is not None else None, meta,
+                                  cache, ov[:R])
+        if R < T:
+            self._attend_folded(q[R:], qf, g[R:] if g is not None else None,
+                                meta, cache, R, ov[R:])
         return self.o_proj(ov.view(T, H * c.vdim))
 
 

@@ -325,6 +325,8 @@ class MomedraLM(nn.Module):
         for layer in self.layers:
             if layer.routed is not None:
                 layer.routed.invalidate_packed()
+            if isinstance(layer.mixer, LatentAttention):
+                layer.mixer.invalidate_packed()
         return n
 
     def expected_tensor_names(self) -> List[str]:

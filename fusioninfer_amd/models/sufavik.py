@@ -307,6 +307,8 @@ class SufavikLM(nn.Module):
         for layer in self.layers:
             if isinstance(layer.mlp, SharedExpertMoE):
                 layer.mlp.routed.invalidate_packed()
+            if isinstance(layer.mixer, LatentAttention):
+                layer.mixer.invalidate_packed()
         return n
 
     def expected_tensor_names(self) -> List[str]:

@@ -38,6 +38,8 @@ void launch_latent_query_rope(A* q_out, const A* q, int64_t q_stride,
                               const int* positions, const float* inv_freq,
                               int rot_pairs, float rot_mult, int T, int H,
                               int D, int R, int C, hipStream_t st);
+void launch_paged_rows_gather(void* out, const void* cache, const int* slots,
+                              int rows, int64_t row_bytes, hipStream_t st);
 template <typename A>
 void launch_silu_and_mul(A* out, const A* gu, int T, int F, hipStream_t st);
 

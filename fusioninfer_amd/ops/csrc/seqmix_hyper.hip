@@ -13,7 +13,10 @@
 //  * latent_query_rope: the trailing rot_dim entries of every query head
 //    rotated into the tail of the folded query buffer; one workgroup per
 //    row, angles computed once for all heads.
+//  * paged_rows_gather: cache rows at given slots, laid end to end.
 //  * silu_and_mul.
+
+#include <type_traits>
 
 #include "seqmix.h"
 #include "seqmix_hyper.h"
@@ -250,8 +253,8 @@ constexpr int kMaxRotPairs = 512;
 
 template <typename A>
 __global__ __launch_bounds__(256) void latent_query_rope_kernel(
-    A* __restrict__ q_out,            // [T, H, C + R]
-    const A* __restrict__ q, int64_t q_stride,        // [T, H*(D+R)]
+    A* q_out,                         // [T, H, C + R]; may be q itself (C = D)
+    const A* q, int64_t q_stride,     // [T, H*(D+R)]
     const int* __restrict__ positions, const float* __restrict__ inv_freq,
     int rot_pairs, float rot_mult, int H, int D, int R, int C) {
   __shared__ float cs_t[kMaxRotPairs], sn_t[kMaxRotPairs];
@@ -279,6 +282,17 @@ __global__ __launch_bounds__(256) void latent_query_rope_kernel(
     Act<A>::st(dst + 2 * i, u);
     Act<A>::st(dst + 2 * i + 1, w);
   }
+}
+
+// rows of `words` elements from the given slots of a paged cache
+template <typename V>
+__global__ __launch_bounds__(256) void paged_rows_gather_kernel(
+    V* __restrict__ out, const V* __restrict__ cache,
+    const int* __restrict__ slots, int rows, int words) {
+  const int64_t i = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
+  if (i >= static_cast<int64_t>(rows) * words) return;
+  const int r = i / words, w = i % words;
+  out[i] = cache[static_cast<int64_t>(slots[r]) * words + w];
 }
 
 template <typename A, int VW>
@@ -377,6 +391,25 @@ void launch_latent_query_rope(A* q_out, const A* q, int64_t q_stride,
   hipLaunchKernelGGL(latent_query_rope_kernel<A>, dim3(T), dim3(256), 0, st,
                      q_out, q, q_stride, positions, inv_freq, rot_pairs,
                      rot_mult, H, D, R, C);
+}
+
+void launch_paged_rows_gather(void* out, const void* cache, const int* slots,
+                              int rows, int64_t row_bytes, hipStream_t st) {
+  if (rows == 0) return;
+  auto blocks = [&](int64_t words) {
+    return dim3(static_cast<unsigned>((rows * words + 255) / 256));
+  };
+  if (row_bytes % 16 == 0)
+    hipLaunchKernelGGL(paged_rows_gather_kernel<float4>,
+                       blocks(row_bytes / 16), dim3(256), 0, st,
+                       static_cast<float4*>(out),
+                       static_cast<const float4*>(cache), slots, rows,
+                       static_cast<int>(row_bytes / 16));
+  else
+    hipLaunchKernelGGL(paged_rows_gather_kernel<u16>, blocks(row_bytes / 2),
+                       dim3(256), 0, st, static_cast<u16*>(out),
+                       static_cast<const u16*>(cache), slots, rows,
+                       static_cast<int>(row_bytes / 2));
 }
 
 template <typename A>

@@ -154,6 +154,19 @@ void latent_query_rope(at::Tensor q_out, at::Tensor q, at::Tensor positions,
                       (int)D, (int)R, (int)C, stream()));
 }
 
+void paged_rows_gather(at::Tensor out, at::Tensor cache, at::Tensor slots) {
+  CHECK_ACT(cache);
+  CHECK_I32(slots);
+  TORCH_CHECK(cache.is_contiguous() && cache.dim() == 4 &&
+              cache.size(1) == 1);
+  TORCH_CHECK(out.is_cuda() && out.is_contiguous() && out.dim() == 2 &&
+              out.scalar_type() == cache.scalar_type() &&
+              out.size(0) == slots.numel() && out.size(1) == cache.size(3));
+  fi::launch_paged_rows_gather(
+      out.data_ptr(), cache.data_ptr(), slots.data_ptr<int>(),
+      (int)slots.numel(), cache.size(3) * cache.element_size(), stream());
+}
+
 void silu_and_mul(at::Tensor out, at::Tensor gu) {
   CHECK_ACT(gu);
   TORCH_CHECK(gu.dim() == 2 && gu.is_contiguous() && gu.size(1) % 2 == 0);
@@ -264,6 +277,8 @@ void register_hyper_ops(pybind11::module& m) {
         "paged cache");
   m.def("latent_query_rope", &latent_query_rope,
         "rotated query parts into the folded query buffer");
+  m.def("paged_rows_gather", &paged_rows_gather,
+        "cache rows at given slots, laid end to end");
   m.def("silu_and_mul", &silu_and_mul, "silu(gate) * up");
   m.def("gated_memory", &gated_memory,
         "matrix memory with exponential gates on slot state");

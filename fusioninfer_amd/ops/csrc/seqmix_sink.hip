@@ -642,7 +642,7 @@ int sink_attention_splits(int max_keys) {
 bool sink_attention_has_tiles(int DK, int DV) {
   return (DK == 64 && DV == 64) || (DK == 96 && DV == 96) ||
          (DK == 128 && DV == 128) || (DK == 112 && DV == 96) ||
-         (DK == 288 && DV == 256);
+         (DK == 192 && DV == 128) || (DK == 288 && DV == 256);
 }
 
 template <typename A>
@@ -674,6 +674,7 @@ bool launch_sink_attention_tiles(A* out, const A* q, const A* k_cache,
   FI_TILE(96, 96, 64, 32, 2, 1)
   FI_TILE(128, 128, 64, 32, 2, 1)
   FI_TILE(112, 96, 64, 32, 2, 1)
+  FI_TILE(192, 128, 32, 32, 2, 1)
   FI_TILE(288, 256, 32, 16, 1, 2)
   FI_TILE(288, 256, 32, 16, 1, 1)
 #undef FI_TILE

@@ -16,6 +16,7 @@ from __future__ import annotations
 
 from typing import Optional
 
+import numpy as np
 import torch
 
 from fusioninfer_amd.ops import seqmix_reference as ref
@@ -432,18 +433,20 @@ SPLIT_ROWS_PER_LAUNCH = 512  # rows per launch of the split attention form
 def sink_paged_attention(q, k_cache, v_cache, seq_bt, row_seq, positions,
                          scale: float, sink=None, value_dims: int = 0,
                          out_gate=None, seq_cu=None, tiles=None,
-                         window: int = 0, keep_first: int = 0):
+                         window: int = 0, keep_first: int = 0, out=None):
     """Causal softmax attention over the paged cache with separate key and
     value sizes, an optional per-head sink in the denominator, values that
     may be the leading ``value_dims`` entries of the cached keys
     (``v_cache`` None) and an optional sigmoid gate on the result, per
     (row, head) ([T, H]) or per entry ([T, H*Dv]). ``window`` > 0 hides
     key j from position p unless p - j < window or j < keep_first.
-    ``tiles`` as for ranged_paged_attention."""
+    ``tiles`` as for ranged_paged_attention; ``out``: contiguous rows to
+    write into."""
     if q.is_cuda:
         T, H, _ = q.shape
         V = v_cache.shape[3] if v_cache is not None else int(value_dims)
-        out = torch.empty((T, H, V), dtype=q.dtype, device=q.device)
+        if out is None:
+            out = torch.empty((T, H, V), dtype=q.dtype, device=q.device)
         tile_seq = tile_row0 = None
         tile_rows = 0
         if (tiles is not None and seq_cu is not None and tiles[2] > 0
@@ -467,9 +470,56 @@ def sink_paged_attention(q, k_cache, v_cache, seq_bt, row_seq, positions,
                                        tile_row0, int(tile_rows), part_ml,
                                        part_o, int(window), int(keep_first))
         return out
-    return ref.sink_paged_attention(q, k_cache, v_cache, seq_bt, row_seq,
-                                    positions, scale, sink, value_dims,
-                                    out_gate, window, keep_first)
+    res = ref.sink_paged_attention(q, k_cache, v_cache, seq_bt, row_seq,
+                                   positions, scale, sink, value_dims,
+                                   out_gate, window, keep_first)
+    if out is not None:
+        res = out.copy_(res)
+    return res
+
+
+def attention_has_tiles(key_dims: int, value_dims: int) -> bool:
+    """sink_paged_attention has a matrix-core tile form for these sizes."""
+    return _native().sink_attention_has_tiles(int(key_dims), int(value_dims))
+
+
+class ContextRows:
+    """The contexts of a step's prompt portions laid end to end: ``slots``
+    [E] int32 cache slot of every context token, ``table`` [groups, longest]
+    int32 its index among the E rows (a block table with blocks of one
+    row)."""
+
+    def __init__(self, spans, block_size: int, device):
+        ends = np.cumsum([c for _, c, _ in spans])
+        self.count = int(ends[-1])
+        slots = np.empty(self.count, dtype=np.int32)
+        table = np.zeros((len(spans), max(c for _, c, _ in spans)),
+                         dtype=np.int32)
+        for i, (_, c, bt) in enumerate(spans):
+            a = int(ends[i]) - c
+            pos = np.arange(c)
+            slots[a: a + c] = (np.asarray(bt, dtype=np.int64)[
+                pos // block_size] * block_size + pos % block_size)
+            table[i, :c] = a + pos
+        self.slots = torch.from_numpy(slots).to(device)
+        self.table = torch.from_numpy(table).to(device)
+
+
+def expansion_pays(spans, rows_per_key: int) -> bool:
+    """Expanding every context row once is cheaper than attending folded
+    when the average context row is read by enough new rows."""
+    ctx = sum(c for _, c, _ in spans)
+    return sum(n * c for n, c, _ in spans) >= rows_per_key * ctx
+
+
+def paged_rows_gather(cache, slots):
+    """Rows of a paged cache [B, 1, bs, N] at the given slots, contiguous."""
+    if cache.is_cuda:
+        out = torch.empty((slots.shape[0], cache.shape[3]),
+                          dtype=cache.dtype, device=cache.device)
+        _native().paged_rows_gather(out, cache, slots)
+        return out
+    return ref.paged_rows_gather(cache, slots)
 
 
 def causal_conv_state(x, conv_w, conv_b, conv_state, seq_cu, row_seq,

@@ -839,6 +839,11 @@ def latent_query_rope_(q, positions, inv_freq, rot_mult: float,
         qr, ang[:, None, :], rot_mult).to(q_out.dtype)
 
 
+def paged_rows_gather(cache, slots):
+    """Rows of cache [B, 1, bs, N] at the given slots -> [len(slots), N]."""
+    return cache.reshape(-1, cache.shape[-1])[slots.long()]
+
+
 def memory_gates(ilin, flin, i_bias, f_bias, cap: float):
     """(log input gate, log forget gate) [T, H] fp32:
     cap * tanh((i + b) / cap) and log sigmoid(cap * tanh((f + b) / cap))."""
