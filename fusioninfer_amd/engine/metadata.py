@@ -39,9 +39,10 @@ class AttnMetadata:
     # (ops.seqmix.build_attention_tiles); None on all-decode steps
     seq_tiles: Optional[tuple] = None
     # host view of the prefill groups: (new rows, context length after the
-    # step, block ids) per group; and what ops.seqmix.context_rows made of it
+    # step, block ids) per group; and the ops.seqmix.ContextRows made of it,
+    # by window
     prefill_spans: Optional[list] = None
-    context_rows: object = None
+    context_rows: Optional[dict] = None
     # LoRA groups for this step (fusioninfer_amd.lora.LoRABatch) or None
     lora: object = None
 

@@ -37,7 +37,8 @@ model designs assemble them freely:
   latent and the rotated part are cached, the expansions are folded into
   the queries and the attended latents; optional per-head softmax sink,
   queries through a normed latent of their own, blended rotary frequencies,
-  a sigmoid gate per head, and layers that read another layer's latents.
+  a sigmoid gate per head, a sliding window, either pairing of the rotation,
+  and layers that read another layer's latents.
 * ``RGLRUMixer``         real-gated linear recurrent unit behind a short
   causal convolution with block-diagonal gates, times a GELU branch.
 * ``SquaredReluMLP``     down(relu(up x)^2) whose up projection may ride a
@@ -68,6 +69,16 @@ model designs assemble them freely:
 * ``SharedExpertMoE``    routed experts next to a silu-gated shared expert
   whose result is multiplied by one sigmoid gate per token; some router
   outputs may be identity experts.
+* ``NormedHeadAttention``  grouped-query softmax attention with projection
+  biases, a weighted RMS norm per query/key head, half-rotated positions
+  with frequencies stretched for long contexts, an optional 1 in the softmax
+  denominator and values blended with those of an earlier layer.
+* ``SelectiveScanMixer``  selective state-space recurrence (per-channel step
+  sizes, per-token input and read-out vectors) behind a short causal
+  convolution, times a silu gate; fp32 state in the state slots.
+* ``PlainMLP``           down(act(up x)).
+* ``SandwichNormLayer``  x <- x + rms(sublayer(rms(x))): a norm in front of
+  and behind every sublayer, residual sum and both norms in one kernel.
 * ``HyperLayer``         several copies of the stream: a sublayer reads the
   RMS norm of a weighted sum of them, and its result is added to every copy
   while the copies are mixed by a small matrix, all in one kernel with the
@@ -788,8 +799,13 @@ class LatentAttentionConfig:
     rot_original: float = 0.0
     rot_fast: float = 0.0
     rot_slow: float = 0.0
+    rot_half: bool = False   # entry i turns with entry i + rot_dims/2
+                             # instead of its neighbour
+    window: int = 0          # >0: keys only from the last `window` positions
 
     def __post_init__(self):
+        if self.window < 0:
+            raise ValueError("window must not be negative")
         if self.rot_dims < 0:
             self.rot_dims = self.rot_dim
         if self.rot_dim % 2 or self.rot_dims % 2:
@@ -950,11 +966,14 @@ class LatentAttention(nn.Module):
         spans = meta.prefill_spans
         if not spans or meta.seq_tiles is None:
             return False
-        if not seqmix.expansion_pays(spans, self.expand_rows_per_key):
+        if not seqmix.expansion_pays(spans, self.expand_rows_per_key,
+                                     c.window):
             return False
         esize = torch.empty((), dtype=self.dtype).element_size()
         per_row = c.heads * (c.dim + c.rot_dim + c.vdim) * esize
-        if per_row * sum(n for _, n, _ in spans) > self.expand_max_bytes:
+        starts = seqmix.context_starts(spans, c.window)
+        if per_row * sum(n - lo for (_, n, _), lo in zip(
+                spans, starts)) > self.expand_max_bytes:
             return False
         return (self.uk.device.type != "cuda" or seqmix.attention_has_tiles(
             c.dim + c.rot_dim, c.vdim))
@@ -985,22 +1004,24 @@ class LatentAttention(nn.Module):
         R, H, D = q.shape[0], c.heads, c.dim + c.rot_dim
         kv = cache["kv"]
         if meta.context_rows is None:
-            meta.context_rows = seqmix.ContextRows(
-                meta.prefill_spans, kv.shape[2], kv.device)
-        ctx = meta.context_rows
-        pos = meta.positions[:R]
+            meta.context_rows = {}
+        ctx = meta.context_rows.get(c.window)
+        if ctx is None:
+            ctx = meta.context_rows[c.window] = seqmix.ContextRows(
+                meta.prefill_spans, kv.shape[2], kv.device, c.window)
         qh = q.view(R, H, D)
-        seqmix.latent_query_rope_(q, pos, self.inv_freq, self.rot_mult, H,
-                                  c.dim, c.rot_dim, c.dim, qh)
+        seqmix.latent_query_rope_(q, meta.positions[:R], self.inv_freq,
+                                  self.rot_mult, H, c.dim, c.rot_dim, c.dim,
+                                  qh, c.rot_half)
         wk, wv = self._expand_weights()
         rows = seqmix.paged_rows_gather(kv, ctx.slots)
         k = F.linear(rows, wk).view(ctx.count, H, 1, D)
         v = F.linear(rows[:, : c.rank], wv).view(ctx.count, H, 1, c.vdim)
         n = len(meta.prefill_spans)
         seqmix.sink_paged_attention(
-            qh, k, v, ctx.table, meta.row_seq[:R], pos, c.scale,
+            qh, k, v, ctx.table, meta.row_seq[:R], ctx.positions, c.scale,
             sink=self.sink, out_gate=gate, seq_cu=meta.seq_cu[: n + 1],
-            tiles=meta.seq_tiles, out=out)
+            tiles=meta.seq_tiles, window=c.window, out=out)
 
     def _attend_folded(self, q, qf, gate, meta, cache, row0, out):
         """Rows row0.. with the expansions folded around the attention; qf
@@ -1015,7 +1036,7 @@ class LatentAttention(nn.Module):
             qf, cache["kv"], None, meta.seq_bt, meta.row_seq[row0:],
             meta.positions[row0:], c.scale, sink=self.sink,
             value_dims=c.rank, out_gate=gate, seq_cu=meta.seq_cu,
-            tiles=meta.seq_tiles if row0 == 0 else None)
+            tiles=meta.seq_tiles if row0 == 0 else None, window=c.window)
         # expand the attended latents: [H, T, rank] x [H, rank, vdim]
         torch.bmm(o.transpose(0, 1), self.uv_t, out=out.transpose(0, 1))
 
@@ -1030,7 +1051,7 @@ class LatentAttention(nn.Module):
             qf = torch.empty((T - R, H, c.rank + c.rot_dim),
                              dtype=self.dtype, device=self.uk.device)
         if (R == 0 and not c.q_rank and self.own_kv
-                and self.rot_mult == 1.0):
+                and self.rot_mult == 1.0 and not c.rot_half):
             seqmix.latent_rope_cache_(
                 q, dkv, meta.positions, self.inv_freq, self.c_norm, self.eps,
                 cache["kv"], meta.slot_mapping, H, c.dim, c.rot_dim, c.rank,
@@ -1040,13 +1061,14 @@ class LatentAttention(nn.Module):
                 cq = seqmix.latent_norm_cache_(
                     parts.get("dq"), dkv, meta.positions, self.inv_freq,
                     self.rot_mult, self.q_norm, self.c_norm, self.eps,
-                    cache["kv"], meta.slot_mapping, c.rank, c.rot_dim)
+                    cache["kv"], meta.slot_mapping, c.rank, c.rot_dim,
+                    c.rot_half)
                 if c.q_rank:
                     q = self.uq(cq)
             if R < T:
                 seqmix.latent_query_rope_(
                     q[R:], meta.positions[R:], self.inv_freq, self.rot_mult,
-                    H, c.dim, c.rot_dim, c.rank, qf)
+                    H, c.dim, c.rot_dim, c.rank, qf, c.rot_half)
         ov = torch.empty((T, H, c.vdim), dtype=q.dtype, device=q.device)
         if R > 0:
             self._attend_expanded(q[:R].contiguous(),
@@ -1112,6 +1134,25 @@ class RGLRUMixer(nn.Module):
             meta.seq_cu, meta.seq_slots, meta.positions, c.decay_scale,
             self.dtype, max_rows=meta.max_seq_rows)
         return self.o_proj(o)
+
+
+class PlainMLP(nn.Module):
+    """down(act(up x)); ``act`` ("gelu_tanh" or "relu_squared") names the
+    activation."""
+
+    def __init__(self, width: int, ff: int, dtype, act: str = "gelu_tanh"):
+        super().__init__()
+        acts = {"gelu_tanh": seqmix.gelu_tanh,
+                "relu_squared": seqmix.relu_squared}
+        if act not in acts:
+            raise ValueError(f"unsupported activation {act!r}")
+        self.ff = ff
+        self._act = acts[act]
+        self.up_proj = ReplicatedLinear(width, ff, dtype=dtype)
+        self.down_proj = RowParallelLinear(ff, width, dtype=dtype)
+
+    def forward(self, x):
+        return self.down_proj(self._act(self.up_proj(x)))
 
 
 class SquaredReluMLP(nn.Module):
@@ -1487,3 +1528,218 @@ class HyperLayer(nn.Module):
                  else [(self.mlp(h), None, False)])
         return seqmix.hyper_update_(xs, terms, self.hc2_mix, self.hc2_out,
                                     nxt[0], nxt[1], self.eps, self.dtype)
+
+
+# ------------------------------------------------------------------------
+# Family of blocks with a norm in front of and behind every sublayer
+
+
+@dataclasses.dataclass
+class NormedHeadAttentionConfig:
+    heads: int
+    kv_heads: int
+    dim: int                 # per-head query/key size
+    vdim: int                # per-head value size
+    scale: float             # score multiplier
+    rot_dims: int = 0        # leading entries of a head that turn (0: none)
+    rot_base: float = 10000.0
+    # frequencies stretched for long contexts (rot_original 0: none)
+    rot_factor: float = 1.0
+    rot_low: float = 1.0
+    rot_high: float = 1.0
+    rot_original: float = 0.0
+    window: int = 0          # 0: plain causal; else p - j < window
+    one_in_denominator: bool = False   # a sink of score 0 without a value
+    v_mix: bool = False      # values blended with the first such layer's
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if self.rot_dims % 2 or not 0 <= self.rot_dims <= self.dim:
+            raise ValueError("rot.dims must be even and at most dim")
+        if self.window < 0:
+            raise ValueError("window must not be negative")
+
+
+@dataclasses.dataclass
+class SelectiveScanConfig:
+    inner: int               # channels
+    state: int               # states per channel
+    dt_rank: int             # inner size of the step-size projection
+    conv: int                # taps of the causal convolution
+
+    def __post_init__(self):
+        if min(self.inner, self.state, self.dt_rank) < 1:
+            raise ValueError("inner, state and dt_rank must be positive")
+        if self.conv < 1:
+            raise ValueError("conv taps must be >= 1")
+
+
+class NormedHeadAttention(nn.Module):
+    """q, k and v come from the caller's merged projection, with biases; the
+    output projection has a bias too. With ``v_mix`` the layers of a step
+    hand the first one's values on in ``shared``: the first layer leaves its
+    own there, the later ones cache (1 - vmix) v + vmix v_first."""
+
+    has_bias = True
+    biased = ("q", "k", "v")
+
+    def __init__(self, cfg: NormedHeadAttentionConfig, width: int,
+                 eps: float, dtype):
+        super().__init__()
+        self.cfg = cfg
+        self.eps = eps
+        self.dtype = dtype
+        H, G = cfg.heads, cfg.kv_heads
+        self.in_names = ["q", "k", "v"]
+        self.in_sizes = [H * cfg.dim, G * cfg.dim, G * cfg.vdim]
+        self.q_norm = _f32_param((cfg.dim,), 1.0)
+        self.k_norm = _f32_param((cfg.dim,), 1.0)
+        self.vmix = _f32_param((), 0.0) if cfg.v_mix else None
+        self.o_proj = RowParallelLinear(H * cfg.vdim, width, dtype=dtype)
+        self.o_bias = nn.Parameter(torch.zeros(width, dtype=dtype),
+                                   requires_grad=False)
+        self.register_buffer(
+            "inv_freq", seqmix.stretched_rotary(
+                cfg.rot_dims, cfg.rot_base, cfg.rot_factor, cfg.rot_low,
+                cfg.rot_high, cfg.rot_original), persistent=False)
+        self.register_buffer(
+            "sink", torch.zeros(H, dtype=torch.float32)
+            if cfg.one_in_denominator else None, persistent=False)
+
+    def state_tensors(self, num_blocks, block_size, num_slots, device):
+        c = self.cfg
+        return {
+            "k": torch.zeros((num_blocks, c.kv_heads, block_size, c.dim),
+                             dtype=self.dtype, device=device),
+            "v": torch.zeros((num_blocks, c.kv_heads, block_size, c.vdim),
+                             dtype=self.dtype, device=device),
+        }
+
+    def block_bytes(self, block_size: int) -> int:
+        c = self.cfg
+        esize = torch.empty((), dtype=self.dtype).element_size()
+        return c.kv_heads * block_size * (c.dim + c.vdim) * esize
+
+    def forward(self, parts, meta, cache, shared: dict) -> torch.Tensor:
+        q, k, v = parts
+        c = self.cfg
+        v_first = None
+        if c.v_mix:
+            v_first = shared.get("v_first")
+            if v_first is None:
+                shared["v_first"] = v
+        qn = seqmix.headnorm_rope_cache_(
+            q, k, v, v_first, self.vmix, meta.positions, self.q_norm,
+            self.k_norm, self.eps, self.inv_freq, cache["k"], cache["v"],
+            meta.slot_mapping, c.heads, c.kv_heads, c.dim, c.vdim)
+        o = seqmix.sink_paged_attention(
+            qn, cache["k"], cache["v"], meta.seq_bt, meta.row_seq,
+            meta.positions, c.scale, sink=self.sink, seq_cu=meta.seq_cu,
+            tiles=meta.seq_tiles, window=c.window)
+        return F.linear(o.view(o.shape[0], c.heads * c.vdim),
+                        self.o_proj.weight, self.o_bias)
+
+
+class SelectiveScanMixer(nn.Module):
+    """The convolved branch and the gate branch come from the merged
+    projection as one ("in": x rows, then z rows)."""
+
+    has_bias = False
+
+    def __init__(self, cfg: SelectiveScanConfig, width: int, eps: float,
+                 dtype):
+        super().__init__()
+        self.cfg = cfg
+        self.dtype = dtype
+        C = cfg.inner
+        self.in_names, self.in_sizes = ["in"], [2 * C]
+        conv = torch.zeros(C, cfg.conv, dtype=torch.float32)
+        conv[:, -1] = 1.0
+        self.conv_w = nn.Parameter(conv, requires_grad=False)
+        self.conv_b = _f32_param((C,), 0.0)
+        self.x_proj = ReplicatedLinear(C, cfg.dt_rank + 2 * cfg.state,
+                                       dtype=dtype)
+        self.dt_proj = ReplicatedLinear(cfg.dt_rank, C, dtype=dtype)
+        self.dt_bias = _f32_param((C,), 0.0)
+        self.a_log = nn.Parameter(
+            torch.log(torch.arange(1, cfg.state + 1, dtype=torch.float32))
+            .repeat(C, 1), requires_grad=False)
+        self.d_skip = _f32_param((C,), 1.0)
+        self.o_proj = RowParallelLinear(C, width, dtype=dtype)
+
+    def state_tensors(self, num_blocks, block_size, num_slots, device):
+        c = self.cfg
+        return {
+            "conv": torch.zeros((num_slots, max(c.conv - 1, 1), c.inner),
+                                dtype=torch.float32, device=device),
+            "ssm": torch.zeros((num_slots, c.inner, c.state),
+                               dtype=torch.float32, device=device),
+        }
+
+    def block_bytes(self, block_size: int) -> int:
+        return 0
+
+    def forward(self, parts, meta, cache) -> torch.Tensor:
+        xz, = parts
+        c = self.cfg
+        u = seqmix.causal_conv_silu(
+            xz[:, : c.inner], self.conv_w, self.conv_b, cache["conv"],
+            meta.seq_cu, meta.row_seq, meta.seq_slots, meta.positions,
+            max_rows=meta.max_seq_rows)
+        dt, B, C = self.x_proj(u).split([c.dt_rank, c.state, c.state],
+                                        dim=-1)
+        y = seqmix.selective_scan(
+            u, self.dt_proj(dt), self.dt_bias, self.a_log, B, C, self.d_skip,
+            xz[:, c.inner:], cache["ssm"], meta.seq_cu, meta.seq_slots,
+            meta.positions, prefill_spans=meta.prefill_spans)
+        return self.o_proj(y)
+
+
+class SandwichNormLayer(nn.Module):
+    """x <- x + rms(mixer(rms(x) w1)) w1b;  x <- x + rms(ff(rms(x) w2)) w2b
+    on an fp32 stream x. Each residual update is one kernel with the norm
+    behind the sublayer and the norm in front of the next one: ``forward``
+    receives this layer's normed input and the norm weight of what comes
+    next, and returns the next normed input. The mixer's input branches are
+    one merged projection. ``shared``: what the layers of one step hand to
+    each other (mixers with a ``v_mix`` config)."""
+
+    def __init__(self, mixer: nn.Module, mlp: Optional[nn.Module],
+                 width: int, eps: float, dtype):
+        super().__init__()
+        self.mixer = mixer
+        self.mlp = mlp
+        self.eps = eps
+        self.dtype = dtype
+        self.branches: List[str] = list(mixer.in_names)
+        self.sizes: List[int] = list(mixer.in_sizes)
+        self.in_proj = MergedColumnParallelLinear(
+            width, self.sizes, dtype=dtype, bias=mixer.has_bias)
+        self.norm1 = _f32_param((width,), 1.0)
+        self.norm1b = _f32_param((width,), 1.0)
+        if mlp is not None:
+            self.norm2 = _f32_param((width,), 1.0)
+            self.norm2b = _f32_param((width,), 1.0)
+
+    def in_proj_rows(self, branch: str):
+        off = 0
+        for name, size in zip(self.branches, self.sizes):
+            if name == branch:
+                return off, size
+            off += size
+        raise KeyError(branch)
+
+    def forward(self, resid, h, meta, cache, next_norm_w, shared: dict):
+        parts = self.in_proj(h).split(self.sizes, dim=-1)
+        if isinstance(self.mixer, NormedHeadAttention):
+            y = self.mixer(parts, meta, cache, shared)
+        else:
+            y = self.mixer(parts, meta, cache)
+        w_after = self.norm2 if self.mlp is not None else next_norm_w
+        h = seqmix.norm_residual_norm_(resid, y, self.norm1b, w_after,
+                                       self.eps, self.dtype)
+        if self.mlp is None:
+            return h
+        return seqmix.norm_residual_norm_(resid, self.mlp(h), self.norm2b,
+                                          next_norm_w, self.eps, self.dtype)

@@ -293,6 +293,18 @@ def _register_builtin_architectures() -> None:
     register_architecture("Sufavik", sufavik_config, sufavik_model,
                           extensions=("seqmix", "moe"))
 
+    def vatunex_config(raw, model_path):
+        from fusioninfer_amd.models import vatunex
+
+        return vatunex.model_config_from_dict(raw, model_path)
+
+    def vatunex_model(cfg):
+        from fusioninfer_amd.models.vatunex import VatunexLM
+
+        return VatunexLM(cfg)
+
+    register_architecture("Vatunex", vatunex_config, vatunex_model)
+
 
 _register_builtin_architectures()
 

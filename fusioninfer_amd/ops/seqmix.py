@@ -484,32 +484,48 @@ def attention_has_tiles(key_dims: int, value_dims: int) -> bool:
 
 
 class ContextRows:
-    """The contexts of a step's prompt portions laid end to end: ``slots``
-    [E] int32 cache slot of every context token, ``table`` [groups, longest]
-    int32 its index among the E rows (a block table with blocks of one
-    row)."""
+    """What the new rows of a step's prompt portions can see of their
+    contexts, laid end to end: ``slots`` [E] int32 cache slot of every such
+    token, ``table`` [groups, longest] int32 its index among the E rows (a
+    block table with blocks of one row), ``positions`` [new rows] int32
+    where the new rows stand in it. With ``window`` > 0 the tokens before
+    the first new row's window are left out."""
 
-    def __init__(self, spans, block_size: int, device):
-        ends = np.cumsum([c for _, c, _ in spans])
+    def __init__(self, spans, block_size: int, device, window: int = 0):
+        spans = [(n, c, lo, bt) for (n, c, bt), lo in zip(
+            spans, context_starts(spans, window))]
+        ends = np.cumsum([c - lo for _, c, lo, _ in spans])
         self.count = int(ends[-1])
         slots = np.empty(self.count, dtype=np.int32)
-        table = np.zeros((len(spans), max(c for _, c, _ in spans)),
+        table = np.zeros((len(spans), max(c - lo for _, c, lo, _ in spans)),
                          dtype=np.int32)
-        for i, (_, c, bt) in enumerate(spans):
-            a = int(ends[i]) - c
-            pos = np.arange(c)
-            slots[a: a + c] = (np.asarray(bt, dtype=np.int64)[
+        for i, (_, c, lo, bt) in enumerate(spans):
+            a = int(ends[i]) - (c - lo)
+            pos = np.arange(lo, c)
+            slots[a: a + c - lo] = (np.asarray(bt, dtype=np.int64)[
                 pos // block_size] * block_size + pos % block_size)
-            table[i, :c] = a + pos
+            table[i, : c - lo] = a + pos - lo
+        place = np.concatenate([np.arange(c - lo - n, c - lo)
+                                for n, c, lo, _ in spans])
         self.slots = torch.from_numpy(slots).to(device)
         self.table = torch.from_numpy(table).to(device)
+        self.positions = torch.from_numpy(place.astype(np.int32)).to(device)
 
 
-def expansion_pays(spans, rows_per_key: int) -> bool:
-    """Expanding every context row once is cheaper than attending folded
-    when the average context row is read by enough new rows."""
-    ctx = sum(c for _, c, _ in spans)
-    return sum(n * c for n, c, _ in spans) >= rows_per_key * ctx
+def context_starts(spans, window: int):
+    """First context position that a portion's new rows can see."""
+    return [max(c - n - window + 1, 0) if window > 0 else 0
+            for n, c, _ in spans]
+
+
+def expansion_pays(spans, rows_per_key: int, window: int = 0) -> bool:
+    """Expanding every visible context row once is cheaper than attending
+    folded when the average such row is read by enough new rows."""
+    ctx = pairs = 0
+    for (n, c, _), lo in zip(spans, context_starts(spans, window)):
+        ctx += c - lo
+        pairs += n * (min(c, window) if window > 0 else c)
+    return pairs >= rows_per_key * ctx
 
 
 def paged_rows_gather(cache, slots):
@@ -690,9 +706,10 @@ def hyper_update_(xs, terms, mix, w_out, w_in, norm_w, eps: float, out_dtype):
 
 def latent_norm_cache_(dq, dkv, positions, inv_freq, rot_mult: float, q_w,
                        c_w, eps: float, kv_cache, slot_mapping, rank: int,
-                       rot_dim: int):
+                       rot_dim: int, half: bool = False):
     """dq (or None): returned RMS-normed with q_w, contiguous. dkv (or
-    None): [normed latent | rotated part] into the paged cache. Both may be
+    None): [normed latent | rotated part] into the paged cache; ``half``:
+    entry i turns with entry i + n instead of its neighbour. Both may be
     column slices of one projection output."""
     src = dq if dq is not None else dkv
     if src is not None and src.is_cuda:
@@ -701,25 +718,26 @@ def latent_norm_cache_(dq, dkv, positions, inv_freq, rot_mult: float, q_w,
             out = torch.empty(dq.shape, dtype=dq.dtype, device=dq.device)
         _native().latent_norm_cache(out, dq, dkv, positions, inv_freq,
                                     float(rot_mult), q_w, c_w, eps, kv_cache,
-                                    slot_mapping, int(rank), int(rot_dim))
+                                    slot_mapping, int(rank), int(rot_dim),
+                                    bool(half))
         return out
     return ref.latent_norm_cache_(dq, dkv, positions, inv_freq, rot_mult,
                                   q_w, c_w, eps, kv_cache, slot_mapping,
-                                  rank, rot_dim)
+                                  rank, rot_dim, half)
 
 
 def latent_query_rope_(q, positions, inv_freq, rot_mult: float,
                        num_heads: int, dim: int, rot_dim: int, rank: int,
-                       q_out):
+                       q_out, half: bool = False):
     """Rotated trailing part of every query head into q_out[:, :, rank:]
-    ([T, H, rank+rot_dim])."""
+    ([T, H, rank+rot_dim]); ``half`` as for latent_norm_cache_."""
     if q.is_cuda:
         _native().latent_query_rope(q_out, q, positions, inv_freq,
                                     float(rot_mult), num_heads, dim, rot_dim,
-                                    rank)
+                                    rank, bool(half))
         return
     ref.latent_query_rope_(q, positions, inv_freq, rot_mult, num_heads, dim,
-                           rot_dim, rank, q_out)
+                           rot_dim, rank, q_out, half)
 
 
 MEMORY_COLUMNS = 64  # value columns per workgroup of the memory kernels
@@ -763,3 +781,85 @@ def silu_and_mul(gu):
         _native().silu_and_mul(out, gu)
         return out
     return ref.silu_and_mul(gu)
+
+
+# ------------------------------------------------------------------------
+# norm in front of and behind every sublayer, normed heads with half
+# rotation and blended values, selective scan behind a short convolution
+
+stretched_rotary = ref.stretched_rotary
+
+
+def norm_residual_norm_(resid, y, w_post, w_next, eps: float, out_dtype):
+    """resid (fp32, in place) += rms(y) * w_post; returns rms(resid) *
+    w_next, the next sublayer's input."""
+    if resid.is_cuda:
+        out = torch.empty(resid.shape, dtype=out_dtype, device=resid.device)
+        _native().norm_residual_norm(resid, y, w_post, w_next, out, eps)
+        return out
+    return ref.norm_residual_norm_(resid, y, w_post, w_next, eps, out_dtype)
+
+
+def headnorm_rope_cache_(q, k, v, v_first, lam, positions, q_w, k_w,
+                         eps: float, inv_freq, k_cache, v_cache,
+                         slot_mapping, num_heads: int, num_kv_heads: int,
+                         dim: int, vdim: int):
+    """RMS norm of every query/key head with a shared weight, rotation of
+    entry i with entry i + n, keys and values into the paged caches; with
+    ``v_first`` the values are (1 - lam) v + lam v_first (lam: one fp32
+    number on the device). q/k/v/v_first may be column slices of projection
+    outputs; returns a fresh contiguous q [T, H, dim]."""
+    if q.is_cuda:
+        out = torch.empty((q.shape[0], num_heads, dim), dtype=q.dtype,
+                          device=q.device)
+        _native().headnorm_rope_cache(
+            out, q, k, v, v_first, lam if v_first is not None else None,
+            positions, q_w, k_w, eps, inv_freq, k_cache, v_cache,
+            slot_mapping, num_heads, num_kv_heads, dim, vdim)
+        return out
+    return ref.headnorm_rope_cache_(q, k, v, v_first, lam, positions, q_w,
+                                    k_w, eps, inv_freq, k_cache, v_cache,
+                                    slot_mapping, num_heads, num_kv_heads,
+                                    dim, vdim)
+
+
+def gelu_tanh(x):
+    """tanh form of gelu, elementwise on [T, N] rows."""
+    if x.is_cuda:
+        out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+        _native().gelu_tanh(out, x)
+        return out
+    return ref.gelu_tanh(x)
+
+
+def causal_conv_silu(x, conv_w, conv_b, conv_state, seq_cu, row_seq,
+                     seq_slots, positions, max_rows: int = 0):
+    """silu of the causal convolution of x (a column slice is fine), in x's
+    dtype; the tail of every sequence stays in conv_state. ``max_rows``:
+    longest group of the step (0: unknown)."""
+    if x.is_cuda:
+        out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+        _native().causal_conv_silu(out, x, conv_w, conv_b, conv_state,
+                                   seq_cu, row_seq, seq_slots, positions,
+                                   int(max_rows))
+        return out
+    return ref.causal_conv_silu(x, conv_w, conv_b, conv_state, seq_cu,
+                                seq_slots, positions)
+
+
+def selective_scan(u, dt_lin, dt_bias, a_log, B, C, D, z, state, seq_cu,
+                   seq_slots, positions, prefill_spans=None):
+    """Selective state-space recurrence on the slot state [slots, channels,
+    N] fp32, times silu(z); returns [T, channels] in u's dtype.
+    dt_lin/B/C/z may be column slices. ``prefill_spans``: host view of the
+    leading multi-row groups (first entry of each: its rows); rows after
+    them are one-row groups."""
+    if u.is_cuda:
+        out = torch.empty(u.shape, dtype=u.dtype, device=u.device)
+        lens = [int(s[0]) for s in prefill_spans] if prefill_spans else []
+        _native().selective_scan(out, u, dt_lin, dt_bias, a_log, B, C, D, z,
+                                 state, seq_cu, seq_slots, positions,
+                                 len(lens), sum(lens), max(lens, default=0))
+        return out
+    return ref.selective_scan(u, dt_lin, dt_bias, a_log, B, C, D, z, state,
+                              seq_cu, seq_slots, positions)

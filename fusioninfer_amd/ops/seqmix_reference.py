@@ -487,6 +487,18 @@ def _rotate_interleaved(x, ang, mult: float = 1.0):
     return out
 
 
+def _rotate(x, ang, mult: float = 1.0, half: bool = False):
+    """Rotation with either pairing: neighbours (2i, 2i+1), or with
+    ``half`` entry i with entry i + n (n angles)."""
+    if not half:
+        return _rotate_interleaved(x, ang, mult)
+    n = ang.shape[-1]
+    cs, sn = torch.cos(ang) * mult, torch.sin(ang) * mult
+    u, w = x[..., :n], x[..., n:2 * n]
+    return torch.cat([u * cs - w * sn, w * cs + u * sn, x[..., 2 * n:]],
+                     dim=-1)
+
+
 def latent_rope_cache_(q, ckr, positions, inv_freq, norm_w, eps: float,
                        kv_cache, slot_mapping, num_heads: int, dim: int,
                        rot_dim: int, rank: int, q_out):
@@ -806,16 +818,17 @@ def hyper_update_(xs, terms, mix, w_out, w_in, norm_w, eps: float, out_dtype):
 
 def latent_norm_cache_(dq, dkv, positions, inv_freq, rot_mult: float, q_w,
                        c_w, eps: float, kv_cache, slot_mapping, rank: int,
-                       rot_dim: int):
+                       rot_dim: int, half: bool = False):
     """dq [T, q_rank] (or None): returned RMS-normed with q_w. dkv
     [T, rank+rot_dim] (or None): leading part RMS-normed with c_w, trailing
-    part rotated (cos/sin times rot_mult), the row goes to the paged
-    kv_cache [B, 1, bs, rank+rot_dim]."""
+    part rotated (cos/sin times rot_mult; ``half``: entry i turns with entry
+    i + n instead of its neighbour), the row goes to the paged kv_cache
+    [B, 1, bs, rank+rot_dim]."""
     if dkv is not None:
         ang = positions.float()[:, None] * inv_freq.float()[None, :]
         cf = dkv.float()
         row = torch.cat([_rms(cf[:, :rank], eps) * c_w.float(),
-                         _rotate_interleaved(cf[:, rank:], ang, rot_mult)],
+                         _rotate(cf[:, rank:], ang, rot_mult, half)],
                         dim=-1)
         bs = kv_cache.shape[2]
         slots = slot_mapping.long()
@@ -829,14 +842,15 @@ def latent_norm_cache_(dq, dkv, positions, inv_freq, rot_mult: float, q_w,
 
 def latent_query_rope_(q, positions, inv_freq, rot_mult: float,
                        num_heads: int, dim: int, rot_dim: int, rank: int,
-                       q_out):
+                       q_out, half: bool = False):
     """q [T, H*(dim+rot_dim)]: the trailing rot_dim entries of every head
-    turned (cos/sin times rot_mult) into q_out[:, :, rank:]."""
+    turned (cos/sin times rot_mult; ``half`` as above) into
+    q_out[:, :, rank:]."""
     T = q.shape[0]
     ang = positions.float()[:, None] * inv_freq.float()[None, :]
     qr = q.float().reshape(T, num_heads, dim + rot_dim)[:, :, dim:]
-    q_out[:, :, rank:] = _rotate_interleaved(
-        qr, ang[:, None, :], rot_mult).to(q_out.dtype)
+    q_out[:, :, rank:] = _rotate(
+        qr, ang[:, None, :], rot_mult, half).to(q_out.dtype)
 
 
 def paged_rows_gather(cache, slots):
@@ -900,3 +914,104 @@ def silu_and_mul(gu):
     """gu: [T, 2F] (gate | up) -> silu(gate) * up."""
     g, u = gu.float().chunk(2, dim=-1)
     return (torch.nn.functional.silu(g) * u).to(gu.dtype)
+
+
+# ------------------------------------------------------------------------
+# norm in front of and behind every sublayer, normed heads with half
+# rotation and blended values, selective scan behind a short convolution
+
+def norm_residual_norm_(resid, y, w_post, w_next, eps: float, out_dtype):
+    """resid (fp32, in place) += rms(y) * w_post; returns
+    rms(resid) * w_next."""
+    resid += _rms(y.float(), eps) * w_post.float()
+    return (_rms(resid, eps) * w_next.float()).to(out_dtype)
+
+
+def stretched_rotary(dims: int, base: float, factor: float = 1.0,
+                     low: float = 1.0, high: float = 1.0,
+                     original: float = 0.0):
+    """[dims/2] fp32 angular frequencies base^(-2i/dims). With ``original``
+    > 0: a pair that makes fewer than ``low`` turns over ``original``
+    positions is slowed down by ``factor``, one that makes more than
+    ``high`` turns is kept, in between both are blended linearly in the
+    number of turns."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    f = torch.pow(torch.tensor(float(base), dtype=torch.float64),
+                  -2.0 * i / max(dims, 1))
+    if original:
+        turns = original * f / (2.0 * math.pi)
+        if high > low:
+            s = ((turns - low) / (high - low)).clamp(0.0, 1.0)
+        else:
+            s = (turns >= low).double()
+        f = (1.0 - s) * f / factor + s * f
+    return f.float()
+
+
+def headnorm_rope_cache_(q, k, v, v_first, lam, positions, q_w, k_w,
+                         eps: float, inv_freq, k_cache, v_cache,
+                         slot_mapping, num_heads: int, num_kv_heads: int,
+                         dim: int, vdim: int):
+    """Every query/key head RMS-normed with a weight [dim] shared by the
+    heads, then the first 2n entries (n = len(inv_freq)) turned, entry i
+    with entry i + n. Keys go into the paged k cache, values into the v
+    cache; with ``v_first`` [T, G*vdim] the values are
+    (1 - lam) v + lam v_first. Returns q [T, H, dim]."""
+    T = q.shape[0]
+    ang = (positions.float()[:, None] * inv_freq.float()[None, :])[:, None, :]
+
+    def turn(x, w, heads):
+        x = _rms(x.float().reshape(T, heads, dim), eps) * w.float()
+        return _rotate(x, ang, 1.0, True)
+
+    kn = turn(k, k_w, num_kv_heads)
+    vv = v.float()
+    if v_first is not None:
+        a = lam.float()
+        vv = (1.0 - a) * vv + a * v_first.float()
+    bs = k_cache.shape[2]
+    slots = slot_mapping.long()
+    ok = slots >= 0
+    k_cache[slots[ok] // bs, :, slots[ok] % bs, :] = kn[ok].to(k_cache.dtype)
+    v_cache[slots[ok] // bs, :, slots[ok] % bs, :] = vv.reshape(
+        T, num_kv_heads, vdim)[ok].to(v_cache.dtype)
+    return turn(q, q_w, num_heads).to(q.dtype)
+
+
+def causal_conv_silu(x, conv_w, conv_b, conv_state, seq_cu, seq_slots,
+                     positions):
+    """silu of ``causal_conv_state``, in x's dtype."""
+    return torch.nn.functional.silu(causal_conv_state(
+        x, conv_w, conv_b, conv_state, seq_cu, seq_slots,
+        positions)).to(x.dtype)
+
+
+def selective_scan(u, dt_lin, dt_bias, a_log, B, C, D, z, state, seq_cu,
+                   seq_slots, positions):
+    """Per channel c and state n, with dt = softplus(dt_lin + dt_bias) and
+    A = -exp(a_log):
+
+        S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c u_c B_n
+        out_c = (sum_n S[c, n] C_n + D_c u_c) * silu(z_c).
+
+    ``state`` [slots, channels, N] fp32 carries S (zero at position 0).
+    Returns [T, channels] in u's dtype."""
+    T, W = u.shape
+    uf, Bf, Cf = u.float(), B.float(), C.float()
+    dt = torch.nn.functional.softplus(dt_lin.float() + dt_bias.float())
+    A = -torch.exp(a_log.float())
+    y = torch.empty(T, W, dtype=torch.float32)
+    cu, slots, pos = seq_cu.tolist(), seq_slots.tolist(), positions.tolist()
+    for s in range(len(slots)):
+        t0, t1 = cu[s], cu[s + 1]
+        if t1 <= t0:
+            continue
+        S = _group_state(state, slots[s], pos[t0], tuple(A.shape))
+        for t in range(t0, t1):
+            S = (torch.exp(dt[t][:, None] * A) * S
+                 + (dt[t] * uf[t])[:, None] * Bf[t][None, :])
+            y[t] = S @ Cf[t]
+        if slots[s] >= 0:
+            state[slots[s]] = S
+    y = y + D.float() * uf
+    return (y * torch.nn.functional.silu(z.float())).to(u.dtype)
