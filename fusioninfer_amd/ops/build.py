@@ -56,11 +56,15 @@ SEQMIX_SOURCES = [
     "seqmix_hyper.hip",
     "seqmix_memory.hip",
     "seqmix_hyper_bindings.hip",
+    "seqmix_sandwich.hip",
+    "seqmix_scan.hip",
+    "seqmix_scan_bindings.hip",
 ]
 
 EXTENSIONS = {
     "core": ("_C", SOURCES, ["common.h"]),
-    "seqmix": ("_C_seqmix", SEQMIX_SOURCES, ["common.h", "seqmix.h", "seqmix_bind.h", "seqmix_hyper.h"]),
+    "seqmix": ("_C_seqmix", SEQMIX_SOURCES, ["common.h", "seqmix.h", "seqmix_bind.h",
+                "seqmix_hyper.h", "seqmix_scan.h"]),
     "moe": ("_C_moe", MOE_SOURCES, ["common.h", "seqmix.h"]),
 }
 

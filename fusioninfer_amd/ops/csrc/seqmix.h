@@ -88,6 +88,26 @@ FI_DEV void block_reduce_sum2_256(float& a, float& b, float* scratch) {
   b = scratch[4] + scratch[5] + scratch[6] + scratch[7];
 }
 
+template <int CTRL>
+FI_DEV float dpp_move(float x) {
+  return __builtin_bit_cast(
+      float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), CTRL,
+                                         0xF, 0xF, true));
+}
+
+// sum over groups of SL adjacent lanes (a power of two up to 64); every
+// lane of a group ends with the total
+template <int SL>
+FI_DEV float slice_sum(float x) {
+  if (SL >= 2) x += dpp_move<0xB1>(x);     // quad_perm [1,0,3,2]
+  if (SL >= 4) x += dpp_move<0x4E>(x);     // quad_perm [2,3,0,1]
+  if (SL >= 8) x += dpp_move<0x141>(x);    // row_half_mirror: other quad
+  if (SL >= 16) x += dpp_move<0x140>(x);   // row_mirror: other half row
+  if (SL >= 32) x += __shfl_xor(x, 16, 64);
+  if (SL >= 64) x += __shfl_xor(x, 32, 64);
+  return x;
+}
+
 FI_DEV float sigmoidf_acc(float x) { return 1.0f / (1.0f + expf(-x)); }
 
 }  // namespace fi

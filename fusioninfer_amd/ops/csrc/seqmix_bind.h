@@ -38,6 +38,15 @@ inline void check_rows(const at::Tensor& t, int64_t T, int64_t n, const char* wh
               what, ": expected [", T, ", ", n, "] with dense rows");
 }
 
+inline void check_groups(const at::Tensor& seq_cu, const at::Tensor& seq_slots,
+                  const at::Tensor& positions, int64_t T) {
+  CHECK_I32(seq_cu);
+  CHECK_I32(seq_slots);
+  CHECK_I32(positions);
+  TORCH_CHECK(seq_cu.numel() == seq_slots.numel() + 1);
+  TORCH_CHECK(positions.numel() == T);
+}
+
 #define DISPATCH_ACT(t, ...)                          \
   if ((t).scalar_type() == at::kFloat) {              \
     using A = float;                                  \
@@ -54,5 +63,7 @@ A* ptr(const at::Tensor& t) {
 
 }  // namespace fi_bind
 
-// bindings that live in a unit of their own (seqmix_hyper_bindings.hip)
+// bindings that live in units of their own (seqmix_hyper_bindings.hip,
+// seqmix_scan_bindings.hip)
 void register_hyper_ops(pybind11::module& m);
+void register_scan_ops(pybind11::module& m);

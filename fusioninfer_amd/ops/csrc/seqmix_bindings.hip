@@ -236,15 +236,6 @@ void dual_norm_combine_residual(at::Tensor resid, at::Tensor yl, at::Tensor yr,
 // group tables: seq_cu [S+1] ascending from 0 to T, row_seq [T],
 // positions [T], seq_slots [S] < num_slots. Values are produced by the
 // model runner; sizes are checked here.
-void check_groups(const at::Tensor& seq_cu, const at::Tensor& seq_slots,
-                  const at::Tensor& positions, int64_t T) {
-  CHECK_I32(seq_cu);
-  CHECK_I32(seq_slots);
-  CHECK_I32(positions);
-  TORCH_CHECK(seq_cu.numel() == seq_slots.numel() + 1);
-  TORCH_CHECK(positions.numel() == T);
-}
-
 void norm_token_shift(at::Tensor out, at::Tensor resid, at::Tensor g,
                       at::Tensor shift, at::Tensor state, at::Tensor seq_cu,
                       at::Tensor row_seq, at::Tensor positions,
@@ -1283,6 +1274,7 @@ void tanh_cap(at::Tensor x, double cap) {
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   register_hyper_ops(m);
+  register_scan_ops(m);
   m.def("pair_embed", &pair_embed,
         "embedding times a constant plus a (previous id, id) table row; the "
         "previous id of a group's first row lives in a slot state");

@@ -33,24 +33,6 @@
 
 namespace fi {
 
-template <int CTRL>
-FI_DEV float dpp_move(float x) {
-  return __builtin_bit_cast(
-      float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), CTRL,
-                                         0xF, 0xF, true));
-}
-
-// sum over the SL adjacent lanes that hold one column (SL = 4, 8, 16);
-// every lane of the group ends with the total
-template <int SL>
-FI_DEV float slice_sum(float x) {
-  x += dpp_move<0xB1>(x);              // quad_perm [1,0,3,2]
-  x += dpp_move<0x4E>(x);              // quad_perm [2,3,0,1]
-  if (SL >= 8) x += dpp_move<0x141>(x);   // row_half_mirror: other quad
-  if (SL == 16) x += dpp_move<0x140>(x);  // row_mirror: other half row
-  return x;
-}
-
 // vecs[t][head][0..4][DK] = (w, a*u, u, k, r); entries >= dim are the
 // identity (w = 1, rest 0) so padded state rows stay zero
 template <typename A>

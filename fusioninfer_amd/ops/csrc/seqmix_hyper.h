@@ -32,12 +32,12 @@ void launch_latent_norm_cache(A* q_out, const A* dq, int64_t dq_stride, int Q,
                               int rot_pairs, float rot_mult, const float* q_w,
                               const float* c_w, float eps, A* kv_cache,
                               const int* slot_mapping, int T, int C, int R,
-                              int bs, hipStream_t st);
+                              int half, hipStream_t st);
 template <typename A>
 void launch_latent_query_rope(A* q_out, const A* q, int64_t q_stride,
                               const int* positions, const float* inv_freq,
                               int rot_pairs, float rot_mult, int T, int H,
-                              int D, int R, int C, hipStream_t st);
+                              int D, int R, int C, int half, hipStream_t st);
 void launch_paged_rows_gather(void* out, const void* cache, const int* slots,
                               int rows, int64_t row_bytes, hipStream_t st);
 template <typename A>

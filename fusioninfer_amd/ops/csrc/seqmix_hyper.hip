@@ -8,8 +8,9 @@
 //    the next sublayer's input rms(sum_s a_s x_s) * w from the new copies:
 //    the copies are read once and written once.
 //  * latent_norm_cache: RMS norm of the query latent to a dense buffer; RMS
-//    norm of the key/value latent and rotation of the shared key part into
-//    one paged cache row. One wave per (row, part).
+//    norm of the key/value latent and rotation of the shared key part (pairs
+//    of neighbours, or entry i with entry i + n) into one paged cache row.
+//    One wave per (row, part).
 //  * latent_query_rope: the trailing rot_dim entries of every query head
 //    rotated into the tail of the folded query buffer; one workgroup per
 //    row, angles computed once for all heads.
@@ -220,7 +221,7 @@ __global__ __launch_bounds__(256) void latent_norm_cache_kernel(
     const int* __restrict__ positions, const float* __restrict__ inv_freq,
     int rot_pairs, float rot_mult, const float* __restrict__ q_w,
     const float* __restrict__ c_w, float eps, A* __restrict__ kv_cache,
-    const int* __restrict__ slot_mapping, int T, int C, int R, int bs) {
+    const int* __restrict__ slot_mapping, int T, int C, int R, int half) {
   const int lane = threadIdx.x % 64;
   const int64_t t = static_cast<int64_t>(blockIdx.x) * 4 + threadIdx.x / 64;
   if (t >= T) return;
@@ -237,14 +238,15 @@ __global__ __launch_bounds__(256) void latent_norm_cache_kernel(
   row += C;
   const float pos = static_cast<float>(positions[t]);
   for (int i = lane; i < rot_pairs; i += 64) {
-    const float u = Act<A>::ld(src + 2 * i);
-    const float w = Act<A>::ld(src + 2 * i + 1);
+    const int i0 = half ? i : 2 * i, i1 = half ? i + rot_pairs : i0 + 1;
+    const float u = Act<A>::ld(src + i0);
+    const float w = Act<A>::ld(src + i1);
     float sn, cs;
     sincosf(pos * inv_freq[i], &sn, &cs);
     sn *= rot_mult;
     cs *= rot_mult;
-    Act<A>::st(row + 2 * i, u * cs - w * sn);
-    Act<A>::st(row + 2 * i + 1, w * cs + u * sn);
+    Act<A>::st(row + i0, u * cs - w * sn);
+    Act<A>::st(row + i1, w * cs + u * sn);
   }
   for (int d = 2 * rot_pairs + lane; d < R; d += 64) row[d] = src[d];
 }
@@ -256,7 +258,7 @@ __global__ __launch_bounds__(256) void latent_query_rope_kernel(
     A* q_out,                         // [T, H, C + R]; may be q itself (C = D)
     const A* q, int64_t q_stride,     // [T, H*(D+R)]
     const int* __restrict__ positions, const float* __restrict__ inv_freq,
-    int rot_pairs, float rot_mult, int H, int D, int R, int C) {
+    int rot_pairs, float rot_mult, int H, int D, int R, int C, int by_half) {
   __shared__ float cs_t[kMaxRotPairs], sn_t[kMaxRotPairs];
   const int64_t t = blockIdx.x;
   const float pos = static_cast<float>(positions[t]);
@@ -272,15 +274,18 @@ __global__ __launch_bounds__(256) void latent_query_rope_kernel(
     const int hh = it / half, i = it % half;
     const A* src = q + t * q_stride + static_cast<int64_t>(hh) * (D + R) + D;
     A* dst = q_out + (t * H + hh) * (C + R) + C;
-    float u = Act<A>::ld(src + 2 * i);
-    float w = Act<A>::ld(src + 2 * i + 1);
+    // pairs past the turning ones are neighbours in either pairing
+    const bool apart = by_half && i < rot_pairs;
+    const int i0 = apart ? i : 2 * i, i1 = apart ? i + rot_pairs : i0 + 1;
+    float u = Act<A>::ld(src + i0);
+    float w = Act<A>::ld(src + i1);
     if (i < rot_pairs) {
       const float a = u * cs_t[i] - w * sn_t[i];
       w = w * cs_t[i] + u * sn_t[i];
       u = a;
     }
-    Act<A>::st(dst + 2 * i, u);
-    Act<A>::st(dst + 2 * i + 1, w);
+    Act<A>::st(dst + i0, u);
+    Act<A>::st(dst + i1, w);
   }
 }
 
@@ -362,7 +367,7 @@ void launch_latent_norm_cache(A* q_out, const A* dq, int64_t dq_stride, int Q,
                               int rot_pairs, float rot_mult, const float* q_w,
                               const float* c_w, float eps, A* kv_cache,
                               const int* slot_mapping, int T, int C, int R,
-                              int bs, hipStream_t st) {
+                              int half, hipStream_t st) {
   if (T == 0) return;
   auto fits = [](const void* p, int64_t stride) {
     return p == nullptr ||
@@ -376,7 +381,7 @@ void launch_latent_norm_cache(A* q_out, const A* dq, int64_t dq_stride, int Q,
   hipLaunchKernelGGL((latent_norm_cache_kernel<A, VW_>), grid, dim3(256), 0,   \
                      st, q_out, dq, dq_stride, Q, dkv, dkv_stride, positions,  \
                      inv_freq, rot_pairs, rot_mult, q_w, c_w, eps, kv_cache,   \
-                     slot_mapping, T, C, R, bs)
+                     slot_mapping, T, C, R, half)
   if (vec) FI_LAT(4);
   else FI_LAT(1);
 #undef FI_LAT
@@ -386,11 +391,11 @@ template <typename A>
 void launch_latent_query_rope(A* q_out, const A* q, int64_t q_stride,
                               const int* positions, const float* inv_freq,
                               int rot_pairs, float rot_mult, int T, int H,
-                              int D, int R, int C, hipStream_t st) {
+                              int D, int R, int C, int half, hipStream_t st) {
   if (T == 0 || R == 0) return;
   hipLaunchKernelGGL(latent_query_rope_kernel<A>, dim3(T), dim3(256), 0, st,
                      q_out, q, q_stride, positions, inv_freq, rot_pairs,
-                     rot_mult, H, D, R, C);
+                     rot_mult, H, D, R, C, half);
 }
 
 void launch_paged_rows_gather(void* out, const void* cache, const int* slots,
@@ -436,7 +441,8 @@ void launch_silu_and_mul(A* out, const A* gu, int T, int F, hipStream_t st) {
       int, int, hipStream_t);                                                  \
   template void launch_latent_query_rope<A>(A*, const A*, int64_t, const int*, \
                                             const float*, int, float, int,     \
-                                            int, int, int, int, hipStream_t);  \
+                                            int, int, int, int, int,           \
+                                            hipStream_t);                      \
   template void launch_silu_and_mul<A>(A*, const A*, int, int, hipStream_t);
 FI_INST(float)
 FI_INST(u16)

@@ -89,7 +89,8 @@ void latent_norm_cache(OptTensor q_out, OptTensor dq, OptTensor dkv,
                        at::Tensor positions, at::Tensor inv_freq,
                        double rot_mult, OptTensor q_w, OptTensor c_w,
                        double eps, at::Tensor kv_cache,
-                       at::Tensor slot_mapping, int64_t C, int64_t R) {
+                       at::Tensor slot_mapping, int64_t C, int64_t R,
+                       bool half) {
   CHECK_I32(positions);
   CHECK_I32(slot_mapping);
   CHECK_F32(inv_freq);
@@ -130,12 +131,12 @@ void latent_norm_cache(OptTensor q_out, OptTensor dq, OptTensor dkv,
       dq.has_value() ? q_w->data_ptr<float>() : nullptr,
       dkv.has_value() ? c_w->data_ptr<float>() : nullptr, (float)eps,
       ptr<A>(kv_cache), slot_mapping.data_ptr<int>(), (int)T, (int)C, (int)R,
-      (int)kv_cache.size(2), stream()));
+      (int)half, stream()));
 }
 
 void latent_query_rope(at::Tensor q_out, at::Tensor q, at::Tensor positions,
                        at::Tensor inv_freq, double rot_mult, int64_t H,
-                       int64_t D, int64_t R, int64_t C) {
+                       int64_t D, int64_t R, int64_t C, bool half) {
   CHECK_ACT(q);
   CHECK_I32(positions);
   CHECK_F32(inv_freq);
@@ -151,7 +152,7 @@ void latent_query_rope(at::Tensor q_out, at::Tensor q, at::Tensor positions,
                       ptr<A>(q_out), ptr<A>(q), q.stride(0),
                       positions.data_ptr<int>(), inv_freq.data_ptr<float>(),
                       (int)inv_freq.numel(), (float)rot_mult, (int)T, (int)H,
-                      (int)D, (int)R, (int)C, stream()));
+                      (int)D, (int)R, (int)C, (int)half, stream()));
 }
 
 void paged_rows_gather(at::Tensor out, at::Tensor cache, at::Tensor slots) {

@@ -452,6 +452,17 @@ void launch_latent_rope_cache(A* q_out, const A* q, int64_t q_stride,
 }
 
 template <typename A>
+void launch_conv_tail_update(const A* x, int64_t x_stride, float* conv_state,
+                             const int* seq_cu, const int* seq_slots,
+                             const int* positions, int S, int C, int taps,
+                             int hist, hipStream_t st) {
+  if (S == 0 || taps <= 1) return;
+  hipLaunchKernelGGL(conv_tail_update_kernel<A>, dim3(S, ceil_div(C, 256)),
+                     dim3(256), 0, st, x, x_stride, conv_state, seq_cu,
+                     seq_slots, positions, C, taps, hist);
+}
+
+template <typename A>
 void launch_causal_conv_state(float* out, const A* x, int64_t x_stride,
                               const float* conv_w, const float* conv_b,
                               float* conv_state, const int* seq_cu,
@@ -463,10 +474,8 @@ void launch_causal_conv_state(float* out, const A* x, int64_t x_stride,
   hipLaunchKernelGGL(causal_conv_state_kernel<A>, dim3(T, cb), dim3(256), 0,
                      st, out, x, x_stride, conv_w, conv_b, conv_state, seq_cu,
                      row_seq, seq_slots, positions, C, taps, hist);
-  if (taps > 1)
-    hipLaunchKernelGGL(conv_tail_update_kernel<A>, dim3(S, cb), dim3(256), 0,
-                       st, x, x_stride, conv_state, seq_cu, seq_slots,
-                       positions, C, taps, hist);
+  launch_conv_tail_update<A>(x, x_stride, conv_state, seq_cu, seq_slots,
+                             positions, S, C, taps, hist, st);
 }
 
 template <typename A>
@@ -509,6 +518,9 @@ void launch_relu_squared(A* out, const A* x, int64_t x_stride, int T, int N,
 }
 
 #define FI_INST(A)                                                             \
+  template void launch_conv_tail_update<A>(                                    \
+      const A*, int64_t, float*, const int*, const int*, const int*, int, int, \
+      int, int, hipStream_t);                                                  \
   template void launch_cast_layer_norm<A>(float*, A*, const A*, const float*,  \
                                           float, int, int, hipStream_t);       \
   template void launch_concat_cast<A>(A*, const float*, const A*, int, int,    \
