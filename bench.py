@@ -72,22 +72,22 @@ def parse_args():
                         "workload mode; headline stays spec-off)")
     p.add_argument("--mixer-compare", action="store_true",
                    help="instead of the serving benchmark: prefill and "
-                        "decode token throughput of the Sufavik, Kazozen, "
-                        "Momedra, Sefalorn and Pinuvik designs at "
+                        "decode token throughput of the Vatunex, Sufavik, "
+                        "Kazozen, Momedra, Sefalorn and Pinuvik designs at "
                         "real-model layer sizes (random weights) next to the Qwen3-style transformer of "
                         "the same sizes")
     p.add_argument("--mc-sizes", default="2048x16,4096x32",
                    help="WIDTHxHEADS list for --mixer-compare (head dim "
                         "128, kv heads = heads/4, ff = 3*width)")
     p.add_argument("--mc-archs",
-                   default="sufavik,kazozen,momedra,sefalorn,pinuvik,transformer")
+                   default="vatunex,sufavik,kazozen,momedra,sefalorn,pinuvik,transformer")
     p.add_argument("--mc-layers", type=int, default=4)
     p.add_argument("--mc-prompt", type=int, default=2048)
     p.add_argument("--mc-prefill-seqs", type=int, default=4)
     p.add_argument("--mc-decode-batch", type=int, default=64)
     p.add_argument("--mc-chunk", type=int, default=1024,
                    help="attention chunk / window (mask size) of the "
-                        "Pinuvik, Sefalorn and Kazozen layers")
+                        "Pinuvik, Sefalorn, Kazozen and Vatunex layers")
     return p.parse_args()
 
 
@@ -104,6 +104,35 @@ def _mixer_compare_config(arch, width, heads, layers, chunk, vocab=32000):
         mc.hidden_size, mc.num_layers = width, layers
         mc.num_heads, mc.num_kv_heads, mc.head_dim = heads, kv, dim
         mc.intermediate_size, mc.vocab_size = ff, vocab
+        return mc
+    if arch == "vatunex":
+        # windowed latent attention, attention with blended values, the
+        # selective scan (inner = 2 * width, 16 states) and blended
+        # attention again, in turn
+        dense = {"kind": "dense", "ff": ff}
+        unit = [
+            {"type": "latent_attention",
+             "mixer": {"heads": heads, "dim": 96, "rot_dim": 32, "vdim": dim,
+                       "kv_rank": 256, "q_rank": 3 * width // 8,
+                       "scale": dim ** -0.5, "mask": {"size": chunk},
+                       "rot": {"base": 1e6, "dims": 32}}, "mlp": dense},
+            {"type": "attention",
+             "mixer": {"heads": heads, "kv_heads": kv, "dim": dim,
+                       "vdim": dim, "scale": dim ** -0.5, "v_mix": True,
+                       "rot": {"base": 5e5, "dims": dim,
+                               "scaling": {"factor": 8.0, "low": 1.0,
+                                           "high": 4.0, "original": 8192}}},
+             "mlp": dense},
+            {"type": "mamba1",
+             "mixer": {"inner": 2 * width, "state": 16, "conv": 4,
+                       "dt_rank": width // 16}, "mlp": dense},
+        ]
+        raw = {"architecture": "Vatunex", "vocab": vocab, "width": width,
+               "norm": {"eps": 1e-5},
+               "layers": [unit[(i % 4) % 3 + i % 4 // 3] for i in
+                          range(layers)]}
+        mc = model_config_from_dict(raw)
+        mc.name = f"vatunex-{width}x{heads}"
         return mc
     if arch == "sufavik":
         # two copies of the stream; latent attention with a dense and with

@@ -72,13 +72,11 @@ def rotary_frequencies(rot):
 def rotate_half(x, pos, freqs):
     """One vector: entry i turns with entry i + n (n = len(freqs)); entries
     from 2 n on pass."""
-    y = x.clone()
     n = len(freqs)
-    for i, f in enumerate(freqs):
-        c, s = math.cos(pos * f), math.sin(pos * f)
-        y[i] = x[i] * c - x[n + i] * s
-        y[n + i] = x[n + i] * c + x[i] * s
-    return y
+    c = torch.tensor([math.cos(pos * f) for f in freqs], dtype=F64)
+    s = torch.tensor([math.sin(pos * f) for f in freqs], dtype=F64)
+    u, v = x[:n], x[n:2 * n]
+    return torch.cat([u * c - v * s, v * c + u * s, x[2 * n:]])
 
 
 # -------------------------------------------------------------- attention
