@@ -108,6 +108,30 @@ FI_DEV float slice_sum(float x) {
   return x;
 }
 
+// hardware exponential and reciprocal, one ulp each
+constexpr float kLog2e = 1.4426950408889634f;
+FI_DEV float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
+FI_DEV float sigmoid_hw(float x) {
+  return __builtin_amdgcn_rcpf(1.0f + exp2_hw(-kLog2e * x));
+}
+
+// log(1 + e^x) = max(x, 0) + log1p(e), e = exp(-|x|) in (0, 1]; log1p from
+// its area-tangent series 2 (s + s^3/3 + ...), s = e / (2 + e) <= 1/3, so
+// that small values keep their relative accuracy
+FI_DEV float softplus_hw(float x) {
+  const float e = exp2_hw(-kLog2e * fabsf(x));
+  const float s = e * __builtin_amdgcn_rcpf(2.0f + e);
+  const float q = s * s;
+  float p = 2.0f / 13.0f;
+  p = p * q + 2.0f / 11.0f;
+  p = p * q + 2.0f / 9.0f;
+  p = p * q + 2.0f / 7.0f;
+  p = p * q + 2.0f / 5.0f;
+  p = p * q + 2.0f / 3.0f;
+  p = p * q + 2.0f;
+  return fmaxf(x, 0.f) + p * s;
+}
+
 FI_DEV float sigmoidf_acc(float x) { return 1.0f / (1.0f + expf(-x)); }
 
 }  // namespace fi

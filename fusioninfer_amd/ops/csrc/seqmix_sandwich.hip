@@ -209,7 +209,7 @@ __global__ __launch_bounds__(256) void gelu_tanh_kernel(
   for (int e = 0; e < VW; ++e) {
     // 0.5 (1 + tanh(a)) = sigmoid(2 a)
     const float z = v[e];
-    v[e] = z * sigmoidf_acc(1.5957691216057308f *
+    v[e] = z * sigmoid_hw(1.5957691216057308f *
                             (z + 0.044715f * z * z * z));
   }
   stv<A, VW>(out + i, v);

@@ -57,6 +57,7 @@ struct ScanArgs {
   float* state;                   // [slots, W, N]
   const int *seq_cu, *seq_slots, *positions;
   int W, N;
+  int vec;                        // set by the launcher of the row form
 };
 int scan_lanes(int N);            // lanes that share a channel
 // rows per segment when the leading groups' longest one is cut so that the

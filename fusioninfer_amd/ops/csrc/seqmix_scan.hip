@@ -29,28 +29,28 @@ namespace fi {
 
 namespace {
 
-FI_DEV float softplus_f(float z) {
-  return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
-}
-
-FI_DEV float silu_f(float z) { return z * sigmoidf_acc(z); }
+FI_DEV float silu_f(float z) { return z * sigmoid_hw(z); }
 
 // ------------------------------------------------------------ convolution
 
-template <typename A, int VW, int TAPS>
+// ROWS consecutive rows per thread; their inputs are loaded up front
+template <typename A, int VW, int TAPS, int ROWS>
 __global__ __launch_bounds__(256) void causal_conv_silu_kernel(
     A* __restrict__ out, const A* __restrict__ x, int64_t x_stride,
     const float* __restrict__ conv_w, const float* __restrict__ conv_b,
     float* __restrict__ conv_state, const int* __restrict__ seq_cu,
     const int* __restrict__ row_seq, const int* __restrict__ seq_slots,
-    const int* __restrict__ positions, int T, int C, int hist, int rows,
+    const int* __restrict__ positions, int T, int C, int hist,
     int keep_tail) {
   constexpr int HW = TAPS > 1 ? TAPS - 1 : 1;
   const int c = (blockIdx.y * 256 + threadIdx.x) * VW;
   if (c >= C) return;
-  const int t0 = blockIdx.x * rows;
-  const int t1 = min(T, t0 + rows);
-  float w[VW][TAPS], b[VW], win[HW][VW];
+  const int t0 = blockIdx.x * ROWS;
+  float w[VW][TAPS], b[VW], win[HW][VW], xs[ROWS][VW];
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i)
+    ldv<A, VW>(x + static_cast<int64_t>(min(t0 + i, T - 1)) * x_stride + c,
+               xs[i]);
 #pragma unroll
   for (int e = 0; e < VW; ++e) {
     b[e] = conv_b[c + e];
@@ -59,7 +59,11 @@ __global__ __launch_bounds__(256) void causal_conv_silu_kernel(
       w[e][j] = conv_w[static_cast<int64_t>(c + e) * TAPS + j];
   }
   int s = -1;
-  for (int t = t0; t < t1; ++t) {
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    const int t = t0 + i;
+    if (t >= T) return;
+    const float* cur = xs[i];
     const int sn = row_seq[t];
     if (sn != s) {
       // the inputs before this row: earlier rows of the group, then the
@@ -81,8 +85,7 @@ __global__ __launch_bounds__(256) void causal_conv_silu_kernel(
                              C + c, win[j]);
       }
     }
-    float cur[VW], y[VW];
-    ldv<A, VW>(x + static_cast<int64_t>(t) * x_stride + c, cur);
+    float y[VW];
 #pragma unroll
     for (int e = 0; e < VW; ++e) {
       float acc = b[e];
@@ -140,16 +143,25 @@ __global__ __launch_bounds__(256) void causal_conv_silu_any_kernel(
 
 // ------------------------------------------------------------------- scan
 
-constexpr float kLog2e = 1.4426950408889634f;
-
-FI_DEV float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
-
 // four states n0.. of channel c: decay rates in the log2 domain (0 past N)
 FI_DEV void load_rates(const float* a_log, int64_t c, int N, int n0,
                        float* a2) {
 #pragma unroll
   for (int i = 0; i < 4; ++i)
-    a2[i] = n0 + i < N ? -expf(a_log[c * N + n0 + i]) * kLog2e : 0.f;
+    a2[i] = n0 + i < N ? -kLog2e * exp2_hw(kLog2e * a_log[c * N + n0 + i])
+                       : 0.f;
+}
+
+// entries n0.. of a B or C row (0 past N); vec: whole aligned vectors
+template <typename A>
+FI_DEV void load_vector(const A* p, int N, int n0, int vec, float* v) {
+  if (vec && n0 < N) {
+    ldv<A, 4>(p + n0, v);
+    return;
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    v[i] = n0 + i < N ? Act<A>::ld(p + n0 + i) : 0.f;
 }
 
 FI_DEV void load_state(const float* p, int N, int n0, float* S) {
@@ -181,9 +193,9 @@ __global__ __launch_bounds__(256) void selective_scan_portion_kernel(
   constexpr int CH = 256 / LN;             // channels per workgroup
   constexpr int NP = 4 * LN;               // padded states
   constexpr int TB = (LN == 1 || LN >= 32) ? 16 : 32;   // tokens per block
-  constexpr int NE = TB * CH;              // (token, channel) entries
-  constexpr int PT = (NE + 255) / 256;
-  constexpr int BT = (TB * NP + 255) / 256;
+  constexpr int PT = (TB + LN - 1) / LN;   // rows a thread loads and stores
+  constexpr int BR = 256 / NP;             // B / C rows per pass
+  constexpr int BT = (TB + BR - 1) / BR;
   __shared__ float2 s_dt[TB][CH];          // (dt, dt * u)
   __shared__ __attribute__((aligned(16))) float s_b[TB][NP];
   __shared__ __attribute__((aligned(16))) float s_c[TB][NP];
@@ -218,36 +230,37 @@ __global__ __launch_bounds__(256) void selective_scan_portion_kernel(
       load_state(a.state + (static_cast<int64_t>(slot) * a.W + cr) * a.N, a.N,
                  n0, S);
   }
-  // role in loading and storing: entries (row, channel) of a block
+  // role in loading and storing: channel cl, rows rl, rl + LN, ... of a
+  // block. Rows and channels past the end are read from the last ones: rows
+  // get a step size of zero, channels are never stored.
+  const int rl = tid / CH;
+  const int cl = c0 + tid % CH;
+  const bool cok = cl < a.W;
+  const int cm = min(cl, a.W - 1);
+  const int rb = tid / NP;
+  const int km = min(tid % NP, a.N - 1);
+  const float bias = a.dt_bias[cm], skip = a.d_skip[cm];
   A ur[PT], dr[PT], zr[PT], br[BT], cc[BT];
-  float bias[PT], skip[PT];
+  // rows r0, r0 + step, ... of a block from a uniform base pointer and
+  // 32-bit offsets; offsets of rows past the last one fall back to it
+  auto load_rows = [](auto& dst, const A* p, int64_t stride, int r0,
+                      int step, int col, int n) {
+    const unsigned sd = static_cast<unsigned>(stride);
+    const unsigned end = (n - 1) * sd + col;
+    unsigned off = r0 * sd + col;
 #pragma unroll
-  for (int i = 0; i < PT; ++i) {
-    const int c = c0 + (tid + 256 * i) % CH;
-    bias[i] = c < a.W ? a.dt_bias[c] : 0.f;
-    skip[i] = c < a.W ? a.d_skip[c] : 0.f;
-  }
+    for (auto& x : dst) {
+      x = p[min(off, end)];
+      off += step * sd;
+    }
+  };
   auto load_block = [&](int base) {
-#pragma unroll
-    for (int i = 0; i < PT; ++i) {
-      const int e = tid + 256 * i;
-      const int r = base + e / CH, c = c0 + e % CH;
-      ur[i] = dr[i] = A(0);
-      if (e < NE && r < rows && c < a.W) {
-        ur[i] = a.u[(t0 + r) * a.W + c];
-        dr[i] = a.dt[(t0 + r) * a.dts + c];
-      }
-    }
-#pragma unroll
-    for (int i = 0; i < BT; ++i) {
-      const int e = tid + 256 * i;
-      const int r = base + e / NP, k = e % NP;
-      br[i] = cc[i] = A(0);
-      if (e < TB * NP && r < rows && k < a.N) {
-        br[i] = a.B[(t0 + r) * a.bs + k];
-        cc[i] = a.C[(t0 + r) * a.cs + k];
-      }
-    }
+    const int64_t t = t0 + base;
+    const int nt = min(TB, rows - base);
+    load_rows(ur, a.u + t * a.W, a.W, rl, LN, cm, nt);
+    load_rows(dr, a.dt + t * a.dts, a.dts, rl, LN, cm, nt);
+    load_rows(br, a.B + t * a.bs, a.bs, rb, BR, km, nt);
+    load_rows(cc, a.C + t * a.cs, a.cs, rb, BR, km, nt);
   };
   float dt_sum = 0.f;
   load_block(0);
@@ -256,32 +269,25 @@ __global__ __launch_bounds__(256) void selective_scan_portion_kernel(
     float uf[PT];
 #pragma unroll
     for (int i = 0; i < PT; ++i) {
-      const int e = tid + 256 * i;
+      const int e = rl + LN * i;
       uf[i] = Act<A>::ld(&ur[i]);
-      if (e >= NE) continue;
       // rows past the end leave the state alone
       const float dt =
-          e / CH < nt ? softplus_f(Act<A>::ld(&dr[i]) + bias[i]) : 0.f;
-      s_dt[e / CH][e % CH] = float2{dt, dt * uf[i]};
+          e < nt ? softplus_hw(Act<A>::ld(&dr[i]) + bias) : 0.f;
+      if (TB % LN == 0 || e < TB) s_dt[e][tid % CH] = float2{dt, dt * uf[i]};
     }
 #pragma unroll
     for (int i = 0; i < BT; ++i) {
-      const int e = tid + 256 * i;
-      if (e < TB * NP) {
-        s_b[e / NP][e % NP] = Act<A>::ld(&br[i]);
-        s_c[e / NP][e % NP] = Act<A>::ld(&cc[i]);
+      const int e = rb + BR * i;
+      if (TB % BR == 0 || e < TB) {
+        const bool in = tid % NP < a.N;
+        s_b[e][tid % NP] = in ? Act<A>::ld(&br[i]) : 0.f;
+        s_c[e][tid % NP] = in ? Act<A>::ld(&cc[i]) : 0.f;
       }
     }
     __syncthreads();
-    if (pass != kSegmentEnds) {
-#pragma unroll
-      for (int i = 0; i < PT; ++i) {
-        const int e = tid + 256 * i;
-        const int r = base + e / CH, c = c0 + e % CH;
-        zr[i] = A(0);
-        if (e < NE && r < rows && c < a.W) zr[i] = a.z[(t0 + r) * a.zs + c];
-      }
-    }
+    if (pass != kSegmentEnds)
+      load_rows(zr, a.z + (t0 + base) * a.zs, a.zs, rl, LN, cm, nt);
     if (base + TB < rows) load_block(base + TB);
 
     if (pass == kSegmentEnds) {
@@ -298,33 +304,62 @@ __global__ __launch_bounds__(256) void selective_scan_portion_kernel(
         }
       }
     } else {
-      for (int q = 0; q < nt; q += 4) {
+      // operands of four tokens are read while four others are applied
+      struct Four {
+        float2 d[4];
+        float b[4][4], c[4][4];
+      };
+      auto fetch = [&](Four& f, int q) {
 #pragma unroll
         for (int k = 0; k < 4; ++k) {
-          const float2 d = s_dt[q + k][lr];
-          float b4[4], c4[4];
-          ldv<float, 4>(&s_b[q + k][n0], b4);
-          ldv<float, 4>(&s_c[q + k][n0], c4);
-          float y = 0.f;
+          f.d[k] = s_dt[q + k][lr];
+          ldv<float, 4>(&s_b[q + k][n0], f.b[k]);
+          ldv<float, 4>(&s_c[q + k][n0], f.c[k]);
+        }
+      };
+      auto apply = [&](const Four& f, int q) {
+        float y[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+          y[k] = 0.f;
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            S[i] = exp2_hw(d.x * a2[i]) * S[i] + d.y * b4[i];
-            y += S[i] * c4[i];
+            S[i] = exp2_hw(f.d[k].x * a2[i]) * S[i] + f.d[k].y * f.b[k][i];
+            y[k] += S[i] * f.c[k][i];
           }
-          y = slice_sum<LN>(y);
-          if (tid % LN == 0) s_y[q + k][lr] = y;
         }
+        if constexpr (LN == 4) {
+          // four tokens over four lanes: lane l ends with token l's sum
+          const bool o1 = tid & 1, o2 = tid & 2;
+          const float u = (o1 ? y[1] : y[0]) + dpp_move<0xB1>(o1 ? y[0] : y[1]);
+          const float v = (o1 ? y[3] : y[2]) + dpp_move<0xB1>(o1 ? y[2] : y[3]);
+          s_y[q + tid % 4][lr] = (o2 ? v : u) + dpp_move<0x4E>(o2 ? u : v);
+        } else {
+#pragma unroll
+          for (int k = 0; k < 4; ++k) {
+            y[k] = slice_sum<LN>(y[k]);
+            if (tid % LN == 0) s_y[q + k][lr] = y[k];
+          }
+        }
+      };
+      Four even, odd;
+      fetch(even, 0);
+      for (int q = 0; q < nt; q += 8) {
+        fetch(odd, q + 4);
+        apply(even, q);
+        if (q + 8 < nt) fetch(even, q + 8);
+        apply(odd, q + 4);
       }
     }
     __syncthreads();
-    if (pass != kSegmentEnds) {
+    if (pass != kSegmentEnds && cok) {
+      A* op = a.out + (t0 + base) * a.W;
 #pragma unroll
       for (int i = 0; i < PT; ++i) {
-        const int e = tid + 256 * i;
-        const int r = base + e / CH, c = c0 + e % CH;
-        if (e < NE && r < rows && c < a.W)
-          Act<A>::st(a.out + (t0 + r) * a.W + c,
-                     (s_y[e / CH][e % CH] + skip[i] * uf[i]) *
+        const int e = rl + LN * i;
+        if (e < nt)
+          Act<A>::st(op + static_cast<unsigned>(e * a.W + cl),
+                     (s_y[e][tid % CH] + skip * uf[i]) *
                          silu_f(Act<A>::ld(&zr[i])));
       }
     }
@@ -396,19 +431,20 @@ __global__ __launch_bounds__(256) void selective_scan_rows_kernel(
   const float bias = a.dt_bias[c], skip = a.d_skip[c];
   for (int64_t t = first; t < end; ++t) {
     const float u = Act<A>::ld(a.u + t * a.W + c);
-    const float dt = softplus_f(Act<A>::ld(a.dt + t * a.dts + c) + bias);
-    float y = 0.f;
+    const float dt = softplus_hw(Act<A>::ld(a.dt + t * a.dts + c) + bias);
+    const float z = Act<A>::ld(a.z + t * a.zs + c);
+    float y = 0.f, b4[4], c4[4];
+    load_vector(a.B + t * a.bs, a.N, n0, a.vec, b4);
+    load_vector(a.C + t * a.cs, a.N, n0, a.vec, c4);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      if (n0 + i >= a.N) continue;
-      S[i] = exp2_hw(dt * a2[i]) * S[i] +
-             dt * u * Act<A>::ld(a.B + t * a.bs + n0 + i);
-      y += S[i] * Act<A>::ld(a.C + t * a.cs + n0 + i);
+      S[i] = exp2_hw(dt * a2[i]) * S[i] + dt * u * b4[i];
+      y += S[i] * c4[i];
     }
     y = slice_sum<LN>(y);
     if (threadIdx.x % LN == 0)
       Act<A>::st(a.out + t * a.W + c,
-                 (y + skip * u) * silu_f(Act<A>::ld(a.z + t * a.zs + c)));
+                 (y + skip * u) * silu_f(z));
   }
   if (slot >= 0) store_state(sp, a.N, n0, S);
 }
@@ -426,19 +462,19 @@ void launch_causal_conv_silu(A* out, const A* x, int64_t x_stride,
   if (T == 0) return;
   const bool vec = C % 4 == 0 && x_stride % 4 == 0 &&
                    reinterpret_cast<uintptr_t>(x) % (4 * sizeof(A)) == 0;
-  const int rows = T >= 1024 ? 16 : 1;
   const bool fast = taps <= 4;
   const int keep_tail = fast && max_rows == 1;
-#define FI_CONV(VW_, TAPS_)                                                    \
-  hipLaunchKernelGGL((causal_conv_silu_kernel<A, VW_, TAPS_>),                 \
-                     dim3(ceil_div(T, rows), ceil_div(C, 256 * VW_)),          \
+#define FI_CONV(VW_, TAPS_, ROWS_)                                             \
+  hipLaunchKernelGGL((causal_conv_silu_kernel<A, VW_, TAPS_, ROWS_>),          \
+                     dim3(ceil_div(T, ROWS_), ceil_div(C, 256 * VW_)),         \
                      dim3(256), 0, st, out, x, x_stride, conv_w, conv_b,       \
                      conv_state, seq_cu, row_seq, seq_slots, positions, T, C,  \
-                     hist, rows, keep_tail)
+                     hist, keep_tail)
 #define FI_CONV_V(TAPS_)                                                       \
   do {                                                                         \
-    if (vec) FI_CONV(4, TAPS_);                                                \
-    else FI_CONV(1, TAPS_);                                                    \
+    if (vec && T >= 1024) FI_CONV(4, TAPS_, 8);                                \
+    else if (vec) FI_CONV(4, TAPS_, 1);                                        \
+    else FI_CONV(1, TAPS_, 1);                                                 \
   } while (0)
   switch (taps) {
     case 1: FI_CONV_V(1); break;
@@ -517,6 +553,11 @@ void launch_selective_scan_portions(ScanArgs<A> a, int groups, int max_rows,
 template <typename A>
 void launch_selective_scan_rows(ScanArgs<A> a, int s0, int S, hipStream_t st) {
   if (S <= s0) return;
+  auto whole = [](const A* p, int64_t stride) {
+    return reinterpret_cast<uintptr_t>(p) % (4 * sizeof(A)) == 0 &&
+           stride % 4 == 0;
+  };
+  a.vec = a.N % 4 == 0 && whole(a.B, a.bs) && whole(a.C, a.cs);
   const int ln = scan_lanes(a.N);
   FI_LANES(ln, {
     auto kernel = selective_scan_rows_kernel<A, LN>;

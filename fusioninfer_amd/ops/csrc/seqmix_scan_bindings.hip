@@ -176,7 +176,10 @@ void selective_scan(at::Tensor out, at::Tensor u, at::Tensor dt,
               max_rows >= 0 && max_rows <= portion_rows &&
               T - portion_rows == S - groups,
               "rows past the portions must be one-row groups");
+  // grid range, and 32-bit offsets inside a block of 32 rows
   TORCH_CHECK(W <= 65535 * 4);
+  for (const at::Tensor* t : {&dt, &B, &C, &z})
+    TORCH_CHECK(t->stride(0) < (int64_t{1} << 26));
   if (T == 0) return;
   int seg_rows = 0;
   at::Tensor seg_state, seg_dt;
@@ -216,6 +219,7 @@ void selective_scan(at::Tensor out, at::Tensor u, at::Tensor dt,
     a.positions = positions.data_ptr<int>();
     a.W = (int)W;
     a.N = (int)N;
+    a.vec = 0;
     fi::launch_selective_scan_portions<A>(a, (int)groups, (int)max_rows,
                                           seg_rows, ss, sd, stream());
     fi::launch_selective_scan_rows<A>(a, (int)groups, (int)S, stream());

@@ -647,6 +647,43 @@ def test_selective_scan_mixer(device, inner, N, R, taps):
 
 
 @pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("C,taps", [(8, 1), (12, 2), (8, 3), (260, 4),
+                                    (7, 4), (8, 6)])
+@pytest.mark.parametrize("lens", [[500, 3, 2, 531, 1, 1], [9, 2, 1]])
+def test_convolution_over_groups(device, C, taps, lens):
+    """Groups of unequal length side by side (in runs of rows that cross
+    their borders when there are many), each with inputs of an earlier step
+    behind it, then one decoded row each; a wide row's column slice."""
+    g = torch.Generator().manual_seed(C + taps)
+    S = len(lens)
+    first = [2 + s % 3 for s in range(S)]
+    seqs = [torch.randn(first[s] + n + 1, C + 3, generator=g)
+            for s, n in enumerate(lens)]
+    w, b = torch.randn(C, taps, generator=g), torch.randn(C, generator=g)
+    tail = torch.randn(S, max(taps - 1, 1), C, generator=g).to(device)
+    got = [[] for _ in lens]
+    a = [0] * S
+    for count in (first, lens, [1] * S):
+        x = torch.cat([q[a[s]:a[s] + count[s]] for s, q in enumerate(seqs)])
+        cu, pos, rows = [0], [], []
+        for s in range(S):
+            cu.append(cu[-1] + count[s])
+            pos += list(range(a[s], a[s] + count[s]))
+            rows += [s] * count[s]
+        y = seqmix.causal_conv_silu(
+            x.to(device)[:, :C], w.to(device), b.to(device), tail,
+            mk(cu, device), mk(rows, device), mk(list(range(S)), device),
+            mk(pos, device), max_rows=max(count)).cpu()
+        for s in range(S):
+            got[s].append(y[cu[s]:cu[s + 1]])
+            a[s] += count[s]
+    for s, q in enumerate(seqs):
+        want = oracle.silu(oracle.causal_conv(q[:, :C].double(), w.double(),
+                                              b.double()))
+        assert torch.allclose(torch.cat(got[s]).double(), want, atol=1e-4)
+
+
+@pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("lens", [[500, 2, 1, 1], [390, 385], [1100], [2]])
 def test_scan_segments_of_unequal_groups(device, lens):
     """The recurrence alone: groups of unequal length side by side (cut
