@@ -27,7 +27,6 @@ from typing import Dict, Iterable, List, Optional, Tuple, Union
 
 import torch
 import torch.nn as nn
-import torch.nn.functional as F
 
 from fusioninfer_amd.config import ModelConfig
 from fusioninfer_amd.distributed import parallel_state as ps

@@ -7,7 +7,6 @@ Weights use the checkpoint naming (``l<i>.mix.q``, ``l<i>.mix.left.q.b``
 ...), as a dict of float64 tensors; ``cfg`` is the config.json dict.
 """
 
-import math
 
 import torch
 
