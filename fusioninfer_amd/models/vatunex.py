@@ -254,10 +254,16 @@ class VatunexLM(nn.Module):
         """Checkpoint names -> parameters. A mixer's input branches land in
         its layer's merged projection; the layer norms' weights gain the one
         they are stored without; norm weights, step-size biases, decays, skip
-        weights and convolution taps are kept in fp32."""
+        weights and convolution taps are kept in fp32. Second norms of a
+        layer without feed-forward are passed over."""
         n = 0
         seen = set()
+        # norms around a feed-forward that the layer does not have
+        unused = {f"l{i}.norm{q}" for i, layer in enumerate(self.layers)
+                  if layer.mlp is None for q in ("2", "2b")}
         for name, t in tensors:
+            if name in unused:
+                continue
             self._load_one(name, t)
             seen.add(name)
             n += 1
